@@ -1,6 +1,10 @@
-"""Build recipe for libelectrock_moe.so (gfx950 only).
+"""Build recipe for libelectrock_moe.so and libelectrock_decoder.so (gfx950 only).
 
-The library is compiled in-tree with plain hipcc; there is no CPU build of the
+Two libraries, so that a model compiles what it needs: csrc/*.hip is the MoE layer, csrc/decoder/*.hip the kernels of
+decoders with a float32 stream, gated linear attention and latent attention (no hand-counted copies there: the checks
+below are about the first one).
+
+The MoE library is compiled in-tree with plain hipcc; there is no CPU build of the
 kernels and no fallback: importing the ops without the built library fails.
 
 The tiled GEMM kernels copy global memory straight into LDS from inline assembly
@@ -17,11 +21,16 @@ import os
 import re
 import shutil
 import subprocess
+import sys
+import tempfile
+from concurrent.futures import ThreadPoolExecutor
 
 PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 CSRC_DIR = os.path.join(PKG_DIR, "csrc")
 LIB_DIR = os.path.join(PKG_DIR, "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libelectrock_moe.so")
+DECODER_CSRC_DIR = os.path.join(CSRC_DIR, "decoder")
+DECODER_LIB_PATH = os.path.join(LIB_DIR, "libelectrock_decoder.so")
 
 HIPCC_FLAGS = [
     "-O3", "-std=c++17", "--offload-arch=gfx950", "-fPIC", "-shared",
@@ -150,5 +159,51 @@ def build(verbose: bool = False) -> str:
     return LIB_PATH
 
 
+def decoder_sources():
+    return sorted(glob.glob(os.path.join(DECODER_CSRC_DIR, "*.hip")))
+
+
+def build_decoder() -> str:
+    """Compile csrc/decoder/*.hip, side by side, into lib/libelectrock_decoder.so; returns its path."""
+    os.makedirs(LIB_DIR, exist_ok=True)
+    hipcc = hipcc_path()
+    flags = [f for f in HIPCC_FLAGS if f != "-shared" and not f.startswith("-Rpass")]
+    with tempfile.TemporaryDirectory(dir=LIB_DIR) as tmp:
+        def compile_one(src):
+            obj = os.path.join(tmp, os.path.basename(src) + ".o")
+            proc = subprocess.run([hipcc, *flags, "-c", src, "-o", obj], stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+            return obj, proc
+        with ThreadPoolExecutor(max_workers=8) as pool:
+            done = list(pool.map(compile_one, decoder_sources()))
+        log = "\n".join(l for _, p in done for l in p.stdout.splitlines() if "packed-fp32-ops" not in l)
+        if any(p.returncode != 0 for _, p in done):
+            raise RuntimeError("hipcc failed:\n" + log)
+        out = os.path.join(tmp, "lib.so")
+        proc = subprocess.run([hipcc, "--offload-arch=gfx950", "-fPIC", "-shared", *[o for o, _ in done], "-o", out],
+                              stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+        if proc.returncode != 0:
+            raise RuntimeError("hipcc failed to link:\n" + proc.stdout)
+        os.replace(out, DECODER_LIB_PATH)
+    return DECODER_LIB_PATH
+
+
+def ensure_decoder() -> str:
+    """Build the decoder library if it is missing or older than its sources."""
+    deps = decoder_sources() + glob.glob(os.path.join(DECODER_CSRC_DIR, "*.h")) + \
+        [os.path.join(CSRC_DIR, "common.h")] + glob.glob(os.path.join(os.path.dirname(PKG_DIR), "include", "*.h"))
+    if not os.path.exists(DECODER_LIB_PATH) or os.path.getmtime(DECODER_LIB_PATH) < max(map(os.path.getmtime, deps)):
+        build_decoder()
+    return DECODER_LIB_PATH
+
+
+def ensure_moe() -> str:
+    """Build the MoE library if it is missing."""
+    if not os.path.exists(LIB_PATH):
+        build()
+    return LIB_PATH
+
+
 if __name__ == "__main__":
-    print(build(verbose=True))
+    if "decoder" not in sys.argv[1:]:
+        print(build(verbose=True))
+    print(build_decoder())

@@ -1,4 +1,5 @@
-"""ctypes binding of libelectrock_moe.so (the C ABI declared in include/electrock_moe.h).
+"""ctypes binding of libelectrock_moe.so (the C ABI declared in include/electrock_moe.h) and of
+libelectrock_decoder.so (include/electrock_decoder.h).
 
 Nothing here computes: each wrapper turns torch tensors into raw device
 pointers plus the current HIP stream and raises RuntimeError on a non-zero
@@ -7,7 +8,7 @@ status.  There is deliberately no CPU or eager-PyTorch fallback.
 import ctypes
 import os
 
-from ._build import LIB_PATH
+from ._build import DECODER_LIB_PATH, LIB_PATH
 
 # element / index type codes of the C ABI
 DTYPE_F32, DTYPE_BF16, DTYPE_F16 = 0, 1, 2
@@ -40,6 +41,35 @@ EXPORTED_SYMBOLS = (
     "em_moe_forward", "em_moe_forward_gated", "em_gate_topk_softmax", "em_rms_norm", "em_add_rms_norm",
     "em_norm_gate_topk_softmax", "em_moe_forward_normed", "em_moe_forward_static", "em_moe_w2_f16_max_tokens",
 )
+
+
+# every function include/electrock_decoder.h declares
+DECODER_SYMBOLS = (
+    "ed_version", "ed_embed", "ed_residual_norm", "ed_relu_squared", "ed_token_gate", "ed_gla_prefill", "ed_gla_step",
+    "ed_latent_row_elems", "ed_latent_prepare", "ed_latent_paged", "ed_head_gemm", "ed_latent_gather",
+)
+
+
+class GlaArgs(ctypes.Structure):
+    """Mirror of struct ed_gla_args."""
+    _fields_ = ([(n, ctypes.c_void_p) for n in ("q", "k", "v", "g", "a1")] + [("stride", ctypes.c_int64)] +
+                [(n, ctypes.c_void_p) for n in ("a2", "bias", "norm_w", "out", "slots", "starts", "states", "log_decay",
+                                                "chunks", "seq_chunks", "chunk_states", "chunk_decay")] +
+                [(n, ctypes.c_int32) for n in ("n_seqs", "n_chunks", "chunk_tokens", "heads", "dim", "vdim", "rank",
+                                               "a2_stride", "dtype")] +
+                [(n, ctypes.c_float) for n in ("tau", "q_scale", "eps")])
+
+
+class LatentArgs(ctypes.Structure):
+    """Mirror of struct ed_latent_args."""
+    _fields_ = ([("q", ctypes.c_void_p), ("q_stride", ctypes.c_int64), ("down", ctypes.c_void_p),
+                 ("down_stride", ctypes.c_int64)] +
+                [(n, ctypes.c_void_p) for n in ("latent_w", "inv_freq", "positions", "cache_rows", "cache", "q_latent",
+                                                "out", "sink", "q_begin", "starts", "tables", "part_o", "part_ml")] +
+                [("T", ctypes.c_int64)] +
+                [(n, ctypes.c_int32) for n in ("n_seqs", "max_q", "table_width", "block_size", "splits", "heads", "dim",
+                                               "rot", "rank", "dtype")] +
+                [(n, ctypes.c_float) for n in ("scale", "eps")])
 
 
 class MoeLayout(ctypes.Structure):
@@ -109,6 +139,50 @@ def check(code: int, what: str) -> None:
     if code != 0:
         msg = load().em_error_string(code).decode()
         raise RuntimeError(f"{what} failed: {msg} (status {code})")
+
+
+_decoder_lib = None
+
+
+def load_decoder() -> ctypes.CDLL:
+    """Load the built decoder library; raise if it has not been built."""
+    global _decoder_lib
+    if _decoder_lib is not None:
+        return _decoder_lib
+    if not os.path.exists(DECODER_LIB_PATH):
+        raise RuntimeError(
+            f"{DECODER_LIB_PATH} is missing: build it with `python -m electrock_infer_amd._build decoder` "
+            "(there is no fallback implementation)")
+    lib = ctypes.CDLL(DECODER_LIB_PATH)
+    vp, i32, i64, dbl = ctypes.c_void_p, ctypes.c_int, ctypes.c_int64, ctypes.c_double
+    signatures = {
+        "ed_version": [],
+        "ed_embed": [vp, vp, dbl, vp, vp, i64, i64, i32, i32, vp],
+        "ed_residual_norm": [i32, vp, vp, i32, vp, vp, vp, i64, i64, i32, dbl, i32, vp],
+        "ed_relu_squared": [vp, i64, i32, vp],
+        "ed_token_gate": [vp, vp, vp, i64, i32, i64, i32, i32, vp],
+        "ed_gla_prefill": [ctypes.POINTER(GlaArgs), vp],
+        "ed_gla_step": [ctypes.POINTER(GlaArgs), vp],
+        "ed_latent_row_elems": [i32, i32],
+        "ed_latent_prepare": [ctypes.POINTER(LatentArgs), vp],
+        "ed_latent_paged": [ctypes.POINTER(LatentArgs), vp],
+        "ed_head_gemm": [vp, i64, i64, vp, vp, i64, i64, i64, i32, i32, i32, i32, vp],
+        "ed_latent_gather": [vp, vp, i32, i32, vp, vp, i32, i32, i32, vp, i32, vp],
+    }
+    for name, argtypes in signatures.items():
+        fn = getattr(lib, name)
+        fn.restype, fn.argtypes = i32, argtypes
+    _decoder_lib = lib
+    return lib
+
+
+ERROR_TEXT = {-1: "null pointer", -2: "bad shape", -3: "unsupported element type", -4: "unsupported shape or option",
+              -5: "workspace missing or too small", -7: "misaligned pointer"}
+
+
+def check_decoder(code: int, what: str) -> None:
+    if code != 0:
+        raise RuntimeError(f"{what} failed: {ERROR_TEXT.get(code, 'HIP error')} (status {code})")
 
 
 def dtype_code(dtype) -> int:

@@ -1,0 +1,85 @@
+// Shared declarations of the decoder library: float32-stream row kernels, gated linear attention, latent attention.
+#pragma once
+#include "../common.h"
+#include "../../../include/electrock_decoder.h"
+
+namespace em {
+
+__device__ __forceinline__ float silu(float g) { return g / (1.0f + expf(-g)); }
+__device__ __forceinline__ float gelu_tanh(float z) {
+    return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
+// Lets a kernel take `bytes` of dynamic LDS (one CU has 160 KB); 0, or the runtime's error.
+constexpr size_t kLdsPerCu = 160 * 1024;
+inline int allow_lds(const void* kernel, size_t bytes) {
+    if (bytes > kLdsPerCu) return EM_ERR_UNSUPPORTED;
+    if (bytes <= 64 * 1024) return 0;
+    return static_cast<int>(hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(bytes)));
+}
+
+// ---- rows.hip ----
+bool row_width_ok(int W);
+int launch_embed(const int32_t* tokens, const void* table, float scale, float* x, void* copy, int64_t copy_stride,
+                 int64_t T, int W, int dtype, hipStream_t s);
+int launch_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
+                         void* out, int64_t out_stride, int64_t T, int W, float eps, int dtype, hipStream_t s);
+int launch_relu_squared(void* u, int64_t n, int dtype, hipStream_t s);
+int launch_token_gate(void* g, const int32_t* tokens, const void* table, int64_t table_stride, int column0, int64_t T,
+                      int dim, int dtype, hipStream_t s);
+
+// ---- gla.hip ----
+struct GlaProblem {
+    const void *q, *k, *v, *g, *a1;
+    int64_t stride;
+    const void* a2;
+    int rank, a2_stride;
+    const float* bias;
+    float tau;
+    const float* norm_w;
+    void* out;
+    float* bl;
+    const int32_t* chunks;
+    const int32_t *slots, *starts;
+    float *states, *chunk_states, *chunk_decay;
+    int heads, dim, vdim;
+    float q_scale, eps;
+    int dtype;
+};
+bool gla_supported(int heads, int dim, int vdim, int rank);
+int launch_gla_prefill(const GlaProblem& g, const int32_t* seq_chunks, int n_chunks, int n_seqs, int chunk_tokens,
+                       hipStream_t s);
+int launch_gla_step(const GlaProblem& g, int n_seqs, hipStream_t s);
+
+// ---- latent_attention.hip ----
+struct LatentProblem {
+    void* q;                 // projection rows: head h at h * (dim + rot), rotated in place by the prepare step
+    int64_t q_stride;
+    const void* down;        // latent + rotated key part of every token, before norm and rotation
+    int64_t down_stride;
+    const float* latent_w;   // [rank]
+    const float* inv_freq;   // [rot / 2]
+    const int32_t* positions;
+    const int32_t* cache_rows;   // row of the cache that takes every token
+    void* cache;             // [rows, latent_row_elems]
+    const void* q_latent;    // [T, heads, latent_pitch]
+    void* out;               // [T, heads, latent_pitch]
+    const float* sink;       // [heads]
+    const int32_t *q_begin, *starts, *tables;
+    int table_width, block_size;
+    int heads, dim, rot, rank;
+    float scale, eps;
+    int dtype;
+};
+__host__ __device__ constexpr int latent_pitch(int rank) { return (rank + 7) / 8 * 8; }
+__host__ __device__ constexpr int latent_row_elems(int rank, int rot) { return latent_pitch(rank) + (rot + 7) / 8 * 8; }
+bool latent_supported(int heads, int dim, int rot, int rank);
+int launch_latent_prepare(const LatentProblem& p, int64_t T, hipStream_t s);
+int launch_latent_paged(const LatentProblem& p, int n_seqs, int max_q, int splits, float* part_o, float* part_ml,
+                        int64_t T, hipStream_t s);
+int launch_head_gemm(const void* a, int64_t a_row, int64_t a_head, const void* b, void* out, int64_t o_row,
+                     int64_t o_head, int64_t T, int heads, int N, int K, int dtype, hipStream_t s);
+int launch_latent_gather(const void* cache, const int32_t* tables, int table_width, int block_size, const int32_t* k_begin,
+                         const int32_t* k_lens, int n_seqs, int max_k, int row_elems, void* out, int dtype, hipStream_t s);
+
+}  // namespace em

@@ -1,0 +1,176 @@
+// extern "C" surface of libelectrock_decoder.so: argument checks and stage sequencing.
+#include "decoder.h"
+
+using namespace em;
+
+namespace {
+
+inline hipStream_t as_stream(void* s) { return static_cast<hipStream_t>(s); }
+inline bool dtype_ok(int d) { return d == EM_DTYPE_F32 || d == EM_DTYPE_BF16; }
+inline bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+constexpr int64_t kMaxRows = 1 << 24;   // rows of one call: grids and 32-bit row numbers
+constexpr int kMaxSeqs = 65535;
+
+GlaProblem gla_problem(const ed_gla_args& a) {
+    GlaProblem g;
+    g.q = a.q; g.k = a.k; g.v = a.v; g.g = a.g; g.a1 = a.a1;
+    g.stride = a.stride;
+    g.a2 = a.a2; g.rank = a.rank; g.a2_stride = a.a2_stride;
+    g.bias = a.bias; g.tau = a.tau;
+    g.norm_w = a.norm_w; g.out = a.out;
+    g.bl = a.log_decay; g.chunks = a.chunks;
+    g.slots = a.slots; g.starts = a.starts;
+    g.states = a.states; g.chunk_states = a.chunk_states; g.chunk_decay = a.chunk_decay;
+    g.heads = a.heads; g.dim = a.dim; g.vdim = a.vdim;
+    g.q_scale = a.q_scale; g.eps = a.eps; g.dtype = a.dtype;
+    return g;
+}
+
+int check_gla(const ed_gla_args* a) {
+    if (!a) return EM_ERR_NULL_POINTER;
+    if (!dtype_ok(a->dtype)) return EM_ERR_BAD_DTYPE;
+    if (a->n_seqs < 0 || a->n_seqs > kMaxSeqs || a->a2_stride < a->rank || !(a->tau > 0.0f)) return EM_ERR_BAD_SHAPE;
+    if (!gla_supported(a->heads, a->dim, a->vdim, a->rank)) return EM_ERR_UNSUPPORTED;
+    if (a->n_seqs == 0) return 0;
+    if (!a->q || !a->k || !a->v || !a->g || !a->a1 || !a->a2 || !a->bias || !a->norm_w || !a->out || !a->slots ||
+        !a->starts || !a->states)
+        return EM_ERR_NULL_POINTER;
+    if (!aligned16(a->states) || !aligned16(a->chunk_states)) return EM_ERR_ALIGNMENT;
+    return 0;
+}
+
+LatentProblem latent_problem(const ed_latent_args& a) {
+    LatentProblem p;
+    p.q = a.q; p.q_stride = a.q_stride;
+    p.down = a.down; p.down_stride = a.down_stride;
+    p.latent_w = a.latent_w; p.inv_freq = a.inv_freq;
+    p.positions = a.positions; p.cache_rows = a.cache_rows;
+    p.cache = a.cache; p.q_latent = a.q_latent; p.out = a.out; p.sink = a.sink;
+    p.q_begin = a.q_begin; p.starts = a.starts; p.tables = a.tables;
+    p.table_width = a.table_width; p.block_size = a.block_size;
+    p.heads = a.heads; p.dim = a.dim; p.rot = a.rot; p.rank = a.rank;
+    p.scale = a.scale; p.eps = a.eps; p.dtype = a.dtype;
+    return p;
+}
+
+int check_latent(const ed_latent_args* a) {
+    if (!a) return EM_ERR_NULL_POINTER;
+    if (!dtype_ok(a->dtype)) return EM_ERR_BAD_DTYPE;
+    if (a->T < 0 || a->T > kMaxRows) return EM_ERR_BAD_SHAPE;
+    if (!latent_supported(a->heads, a->dim, a->rot, a->rank)) return EM_ERR_UNSUPPORTED;
+    return 0;
+}
+
+}  // namespace
+
+extern "C" {
+
+int ed_version(void) { return 100; }
+
+int ed_embed(const int32_t* tokens, const void* table, double scale, float* x, void* copy, int64_t copy_stride,
+             int64_t T, int W, int dtype, void* stream) {
+    if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
+    if (T < 0 || T > kMaxRows || !row_width_ok(W) || (copy && copy_stride < W)) return EM_ERR_BAD_SHAPE;
+    if (T == 0) return 0;
+    if (!tokens || !table || !x) return EM_ERR_NULL_POINTER;
+    if (!aligned16(table) || !aligned16(x) || (W % 4 == 0 && (reinterpret_cast<uintptr_t>(copy) & 15) % (dtype == EM_DTYPE_F32 ? 16 : 8)))
+        return EM_ERR_ALIGNMENT;
+    return launch_embed(tokens, table, static_cast<float>(scale), x, copy, copy ? copy_stride : W, T, W, dtype, as_stream(stream));
+}
+
+int ed_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
+                     void* out, int64_t out_stride, int64_t T, int W, double eps, int dtype, void* stream) {
+    if (!dtype_ok(dtype) || (update != 0 && y_dtype != dtype && y_dtype != EM_DTYPE_F32)) return EM_ERR_BAD_DTYPE;
+    if (update < 0 || update > 2 || T < 0 || T > kMaxRows || !row_width_ok(W) || (out && out_stride < W)) return EM_ERR_BAD_SHAPE;
+    if (T == 0) return 0;
+    if (!x || (update != 0 && !y) || (update == 1 && !post_w)) return EM_ERR_NULL_POINTER;
+    // rows that are not a multiple of four elements go element by element
+    if (W % 4 == 0 && (!aligned16(x) || !aligned16(y) || !aligned16(post_w) || !aligned16(next_w) || !aligned16(out)))
+        return EM_ERR_ALIGNMENT;
+    return launch_residual_norm(update, x, y, update == 0 ? dtype : y_dtype, post_w, next_w, out, out ? out_stride : W, T, W,
+                                static_cast<float>(eps), dtype, as_stream(stream));
+}
+
+int ed_relu_squared(void* u, int64_t n, int dtype, void* stream) {
+    if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
+    if (n < 0 || n > (int64_t{1} << 38)) return EM_ERR_BAD_SHAPE;
+    if (n == 0) return 0;
+    if (!u) return EM_ERR_NULL_POINTER;
+    if (!aligned16(u)) return EM_ERR_ALIGNMENT;
+    return launch_relu_squared(u, n, dtype, as_stream(stream));
+}
+
+int ed_token_gate(void* g, const int32_t* tokens, const void* table, int64_t table_stride, int column0, int64_t T,
+                  int dim, int dtype, void* stream) {
+    if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
+    if (T < 0 || T > kMaxRows || dim <= 0 || column0 < 0 || column0 + static_cast<int64_t>(dim) > table_stride) return EM_ERR_BAD_SHAPE;
+    if (T == 0) return 0;
+    if (!g || !tokens || !table) return EM_ERR_NULL_POINTER;
+    return launch_token_gate(g, tokens, table, table_stride, column0, T, dim, dtype, as_stream(stream));
+}
+
+int ed_gla_prefill(const ed_gla_args* a, void* stream) {
+    int rc = check_gla(a);
+    if (rc != 0 || a->n_seqs == 0) return rc;
+    if (a->n_chunks < a->n_seqs || a->chunk_tokens <= 0 || a->chunk_tokens % 16 != 0 || a->chunk_tokens / 16 > 65535) return EM_ERR_BAD_SHAPE;
+    if (a->n_chunks > a->n_seqs && (!a->chunk_states || !a->chunk_decay)) return EM_ERR_WORKSPACE;
+    if (!a->log_decay || !a->chunks || !a->seq_chunks) return EM_ERR_NULL_POINTER;
+    if (!aligned16(a->chunks)) return EM_ERR_ALIGNMENT;
+    GlaProblem g = gla_problem(*a);
+    if (a->n_chunks == a->n_seqs) g.chunk_states = nullptr;
+    return launch_gla_prefill(g, a->seq_chunks, a->n_chunks, a->n_seqs, a->chunk_tokens, as_stream(stream));
+}
+
+int ed_gla_step(const ed_gla_args* a, void* stream) {
+    const int rc = check_gla(a);
+    if (rc != 0 || a->n_seqs == 0) return rc;
+    return launch_gla_step(gla_problem(*a), a->n_seqs, as_stream(stream));
+}
+
+int ed_latent_row_elems(int rank, int rot) { return latent_row_elems(rank, rot); }
+
+int ed_latent_prepare(const ed_latent_args* a, void* stream) {
+    const int rc = check_latent(a);
+    if (rc != 0 || a->T == 0) return rc;
+    if (!a->q || !a->down || !a->latent_w || (a->rot > 0 && !a->inv_freq) || !a->positions || !a->cache_rows || !a->cache)
+        return EM_ERR_NULL_POINTER;
+    return launch_latent_prepare(latent_problem(*a), a->T, as_stream(stream));
+}
+
+int ed_latent_paged(const ed_latent_args* a, void* stream) {
+    const int rc = check_latent(a);
+    if (rc != 0 || a->T == 0) return rc;
+    if (a->n_seqs <= 0 || a->n_seqs > kMaxSeqs || a->max_q <= 0 || a->max_q > a->T || a->splits < 1 || a->splits > 65535 ||
+        a->block_size <= 0 || a->table_width <= 0)
+        return EM_ERR_BAD_SHAPE;
+    if (!a->q || !a->q_latent || !a->cache || !a->out || !a->sink || !a->q_begin || !a->starts || !a->tables) return EM_ERR_NULL_POINTER;
+    if (a->splits > 1 && (!a->part_o || !a->part_ml)) return EM_ERR_WORKSPACE;
+    if (!aligned16(a->cache) || !aligned16(a->q_latent)) return EM_ERR_ALIGNMENT;
+    return launch_latent_paged(latent_problem(*a), a->n_seqs, a->max_q, a->splits, a->part_o, a->part_ml, a->T, as_stream(stream));
+}
+
+int ed_head_gemm(const void* a, int64_t a_row, int64_t a_head, const void* b, void* out, int64_t out_row,
+                 int64_t out_head, int64_t T, int heads, int N, int K, int dtype, void* stream) {
+    if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
+    if (T < 0 || T > kMaxRows || heads <= 0 || heads > 65535 || N <= 0 || K <= 0 || a_row < 0 || a_head < 0) return EM_ERR_BAD_SHAPE;
+    if (T == 0) return 0;
+    if (!a || !b || !out) return EM_ERR_NULL_POINTER;
+    if (!aligned16(b)) return EM_ERR_ALIGNMENT;
+    return launch_head_gemm(a, a_row, a_head, b, out, out_row, out_head, T, heads, N, K, dtype, as_stream(stream));
+}
+
+int ed_latent_gather(const void* cache, const int32_t* tables, int table_width, int block_size,
+                     const int32_t* k_begin, const int32_t* k_lens, int n_seqs, int max_k, int row_elems, void* out,
+                     int dtype, void* stream) {
+    if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
+    if (n_seqs < 0 || n_seqs > kMaxSeqs || max_k < 0 || max_k > kMaxRows || row_elems <= 0 || row_elems % 8 != 0 ||
+        block_size <= 0 || table_width <= 0)
+        return EM_ERR_BAD_SHAPE;
+    if (n_seqs == 0 || max_k == 0) return 0;
+    if (!cache || !tables || !k_begin || !k_lens || !out) return EM_ERR_NULL_POINTER;
+    if (!aligned16(cache) || !aligned16(out)) return EM_ERR_ALIGNMENT;
+    return launch_latent_gather(cache, tables, table_width, block_size, k_begin, k_lens, n_seqs, max_k, row_elems, out, dtype,
+                                as_stream(stream));
+}
+
+}  // extern "C"

@@ -5,15 +5,19 @@ from typing import Dict, List, Optional, Sequence as Seq, Union
 
 from .config import EngineConfig, ModelConfig, SamplingParams
 from .model_runner import ModelRunner
+from .registry import load_config
 from .batch_planner import BatchPlanner
 from .sequence import Sequence
 
 
 class LLMEngine:
 
-    def __init__(self, model: Optional[ModelConfig] = None, model_runner=None, **kwargs):
-        """``model_runner``: an object with ``run(seqs, is_prefill[, return_logits])`` to use instead of the GPU model
+    def __init__(self, model: Union[None, str, ModelConfig] = None, model_runner=None, dtype: str = "bfloat16", **kwargs):
+        """``model``: a configuration (random weights) or a model directory with config.json and safetensors files,
+        whose registered architecture decides which model runs, in ``dtype``.  ``model_runner``: an object with ``run(seqs, is_prefill[, return_logits])`` to use instead of the GPU model
         (host tests of the request loop); it must leave ``config.num_kvcache_blocks`` as given."""
+        if isinstance(model, str):
+            kwargs["model_dir"], model = model, load_config(model, dtype)
         self.config = EngineConfig(model=model or ModelConfig(), **kwargs)
         Sequence.block_size = self.config.kvcache_block_size
         self.model_runner = model_runner if model_runner is not None else ModelRunner(self.config)  # sizes config.num_kvcache_blocks
@@ -27,6 +31,8 @@ class LLMEngine:
         limit = self.config.max_model_len          # <= max_position_embeddings: the rotary table ends there
         if len(prompt) + 1 > limit:
             raise ValueError("prompt longer than max_model_len")
+        if len(prompt) and not 0 <= min(prompt) <= max(prompt) < self.config.model.vocab_size:
+            raise ValueError("token id outside the vocabulary")
         seq = Sequence(prompt, sampling_params)
         # no request may grow past the positions the model has: the request ends at max_model_len tokens at the latest
         # (the reference has no such cap, llm_engine.py:88-91; there a long request indexes past its rotary table)
@@ -39,13 +45,14 @@ class LLMEngine:
         positive for a prefill step (tokens in the batch), negative for a decode step (minus the sequences)."""
         plan = self.planner.plan()
         seqs, is_prefill = plan.seqs, plan.is_prefill
+        fed = sum(s.num_scheduled_tokens for s in seqs)
         if self.step_hook is not None:
             token_ids, logits = self.model_runner.run(seqs, is_prefill, return_logits=True)
             self.step_hook(seqs, is_prefill, logits)
         else:
             token_ids = self.model_runner.run(seqs, is_prefill)
         finished = [(seq.seq_id, seq.completion_token_ids) for seq in self.planner.commit(seqs, token_ids)]
-        return finished, (sum(len(s) for s in seqs) if is_prefill else -len(seqs))
+        return finished, (fed if is_prefill else -len(seqs))
 
     def is_finished(self) -> bool:
         return self.planner.idle()

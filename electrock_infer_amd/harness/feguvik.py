@@ -1,0 +1,239 @@
+"""Feguvik: a decoder whose layers mix gated linear attention (recurrent state) and latent attention (paged cache), with
+norms in front of and behind every sublayer, layer scales, a per-layer token input, and a range of layers that runs
+several times with the same weights, each pass with its own cache and state.
+
+The residual stream is float32; projections run in the configuration's compute type (bfloat16, or float32 throughout).
+"""
+from dataclasses import dataclass, field
+from typing import List, Optional, Tuple
+
+import torch
+import torch.nn.functional as F
+from torch import nn
+
+from ..layers.decoder_ops import ADD_NORMED, KEEP, REPLACE, embed_rows, linear_f32, residual_norm
+from ..layers.dense_mlp import DenseMLP
+from ..layers.gla import GatedLinearAttention
+from ..layers.latent_attention import LatentAttention
+from ..layers.token_side import TokenSideInput
+from .batch import RaggedBatch
+
+
+@dataclass
+class LayerSpec:
+    """One entry of config.json's 'layers'; ``ff`` is 0 for a layer without a feed-forward."""
+    kind: str                       # 'gla' | 'latent_attention'
+    mixer: dict
+    ff: int = 0
+    decay_rank: int = 0             # 'gla': inner size of the decay's two factors (not in config.json: a tensor's shape)
+
+
+@dataclass
+class LoopSpec:
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass
+class FeguvikConfig:
+    vocab_size: int
+    width: int
+    layers: List[LayerSpec]
+    norm_eps: float
+    embedding_scale: float = 1.0
+    side_dim: int = 0               # per-layer token input; 0: none
+    loop: Optional[LoopSpec] = None
+    max_position_embeddings: int = 1 << 24      # positions are exact in float32 up to here; there is no table
+    torch_dtype: torch.dtype = field(default=torch.bfloat16)
+
+    @property
+    def has_recurrent_state(self) -> bool:
+        return any(l.kind == "gla" for l in self.layers)
+
+    @classmethod
+    def from_checkpoint(cls, config: dict, shapes: dict, dtype: torch.dtype) -> "FeguvikConfig":
+        layers = []
+        for i, entry in enumerate(config["layers"]):
+            if entry["type"] not in ("gla", "latent_attention"):
+                raise ValueError(f"layer {i}: unknown mixer '{entry['type']}'")
+            mlp = entry.get("mlp")
+            if mlp is not None and mlp["kind"] != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward '{mlp['kind']}'")
+            rot = entry["mixer"].get("rot")
+            if rot is not None and rot["dims"] != entry["mixer"]["rot_dim"]:
+                raise ValueError(f"layer {i}: rot.dims differs from rot_dim")
+            layers.append(LayerSpec(entry["type"], dict(entry["mixer"]), mlp["ff"] if mlp is not None else 0,
+                                    shapes[f"l{i}.mix.a1"][0] if entry["type"] == "gla" else 0))
+        loop, side = config.get("loop"), config.get("token_side")
+        return cls(vocab_size=config["vocab"], width=config["width"], layers=layers, norm_eps=config["norm"]["eps"],
+                   embedding_scale=config["embedding"]["scale"], side_dim=side["dim"] if side else 0,
+                   loop=LoopSpec(loop["start"], loop["stop"], loop["times"]) if loop else None, torch_dtype=dtype)
+
+    def runs(self) -> List[Tuple[int, Optional[int]]]:
+        """(layer, pass or None) in running order."""
+        every = range(len(self.layers))
+        if self.loop is None:
+            return [(i, None) for i in every]
+        a, b = self.loop.start, self.loop.stop
+        return ([(i, None) for i in every[:a]] + [(i, t) for t in range(self.loop.times) for i in every[a:b]] +
+                [(i, None) for i in every[b:]])
+
+
+class FeguvikLayer(nn.Module):
+
+    def __init__(self, cfg: FeguvikConfig, index: int):
+        super().__init__()
+        spec, dtype, m = cfg.layers[index], cfg.torch_dtype, cfg.layers[index].mixer
+        vector = lambda: nn.Parameter(torch.ones(cfg.width, dtype=torch.float32), requires_grad=False)
+        if spec.kind == "gla":
+            self.mix = GatedLinearAttention(cfg.width, m["heads"], m["dim"], m["vdim"], m["tau"], spec.decay_rank,
+                                            cfg.norm_eps, dtype)
+        else:
+            self.mix = LatentAttention(cfg.width, m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], m["scale"],
+                                       m["rot"]["base"], cfg.norm_eps, dtype)
+        self.norm1, self.norm1b, self.ls1 = vector(), vector(), vector()
+        self.mlp = None
+        if spec.ff:
+            self.norm2, self.norm2b, self.ls2 = vector(), vector(), vector()
+            self.mlp = DenseMLP(cfg.width, spec.ff, dtype)
+        self.side = TokenSideInput(cfg.width, cfg.side_dim, index * cfg.side_dim, dtype) if cfg.side_dim else None
+        self.post1 = self.post2 = None
+
+    def finish_loading(self) -> None:
+        """The output norm's weight and the layer scale multiply the same vector: one factor."""
+        self.post1 = (self.norm1b * self.ls1).contiguous()
+        if self.mlp is not None:
+            self.post2 = (self.norm2b * self.ls2).contiguous()
+        if hasattr(self.mix, "finish_loading"):
+            self.mix.finish_loading()
+
+
+class FeguvikForCausalLM(nn.Module):
+
+    ragged_batches = True
+    GLA_CHUNK = 256         # tokens that one workgroup of the linear attention's prompt kernel takes
+
+    def __init__(self, cfg: FeguvikConfig):
+        super().__init__()
+        self.cfg = cfg
+        W, dtype = cfg.width, cfg.torch_dtype
+        matrix = lambda *shape: nn.Parameter(torch.zeros(*shape, dtype=dtype), requires_grad=False)
+        self.embed = matrix(cfg.vocab_size, W)
+        if cfg.side_dim:
+            self.side_embed = matrix(cfg.vocab_size, len(cfg.layers) * cfg.side_dim)
+        if cfg.loop is not None:
+            self.loop_in = matrix(W, 2 * W)
+            self.loop_step = nn.Parameter(torch.zeros(cfg.loop.times, W, dtype=torch.float32), requires_grad=False)
+        self.layers = nn.ModuleList([FeguvikLayer(cfg, i) for i in range(len(cfg.layers))])
+        self.final_norm = nn.Parameter(torch.ones(W, dtype=torch.float32), requires_grad=False)
+        self.head = matrix(cfg.vocab_size, W)
+        self.runs = cfg.runs()
+        self.caches: List[torch.Tensor] = []      # per run: pages of the latent attention or states of the linear one
+        self.layer_hook = None                    # called as hook(run index, stream) behind every layer run when set
+
+    # ---- weights ----
+    _NAMES = {"embed": "embed", "side.embed": "side_embed", "loop.in": "loop_in", "loop.step": "loop_step",
+              "final.norm": "final_norm", "head": "head"}
+
+    def checkpoint_target(self, name: str):
+        """(parameter name, section or None) of a checkpoint tensor, or None."""
+        if name in self._NAMES:
+            return self._NAMES[name], None
+        first, _, rest = name.partition(".")
+        if first[:1] == "l" and first[1:].isdigit() and int(first[1:]) < len(self.layers):
+            prefix = f"layers.{first[1:]}."
+            if not rest.startswith("mix."):
+                return prefix + rest, None
+            entry = self.layers[int(first[1:])].mix.TENSORS.get(rest[4:])
+            if entry is not None:
+                return prefix + "mix." + entry[0], entry[1]
+        return None
+
+    def expected_tensors(self) -> List[str]:
+        """Checkpoint names of every parameter (section)."""
+        cfg, out = self.cfg, ["embed", "final.norm", "head"]
+        out += ["side.embed"] if cfg.side_dim else []
+        out += ["loop.in", "loop.step"] if cfg.loop is not None else []
+        for i, layer in enumerate(self.layers):
+            names = ["norm1", "norm1b", "ls1"] + [f"mix.{n}" for n in layer.mix.TENSORS]
+            names += ["norm2", "norm2b", "ls2", "mlp.up", "mlp.down"] if layer.mlp is not None else []
+            names += ["side.gate", "side.proj", "side.norm"] if layer.side is not None else []
+            out += [f"l{i}.{n}" for n in names]
+        return out
+
+    def finish_loading(self) -> None:
+        for layer in self.layers:
+            layer.finish_loading()
+
+    @torch.no_grad()
+    def init_random_weights(self, seed: int = 0, std: float = 0.02) -> None:
+        """N(0, std) for every matrix, ones for norms and layer scales, zeros for sinks and the decay's bias."""
+        g = torch.Generator(device=self.head.device).manual_seed(seed)
+        for name, p in self.named_parameters():
+            if p.dim() >= 2:
+                p.copy_(torch.randn(p.shape, generator=g, device=p.device, dtype=torch.float32) * std)
+            else:
+                p.fill_(0.0 if name.endswith(("sink", "a2_bias")) else 1.0)
+        self.finish_loading()
+
+    # ---- cache and state ----
+    def cache_bytes(self, block_size: int) -> Tuple[int, int]:
+        """(bytes of a cache block, bytes of a state slot), over all layer runs."""
+        block = slot = 0
+        for i, _ in self.runs:
+            mix = self.layers[i].mix
+            if isinstance(mix, LatentAttention):
+                block += block_size * mix.row_elems() * self.head.element_size()
+            else:
+                slot += mix.heads * mix.dim * mix.vdim * 4
+        return block, slot
+
+    def allocate_cache(self, num_blocks: int, block_size: int, num_slots: int, device) -> None:
+        self.caches = []
+        for i, _ in self.runs:
+            mix = self.layers[i].mix
+            if isinstance(mix, LatentAttention):
+                self.caches.append(torch.zeros(num_blocks, block_size, mix.row_elems(), dtype=self.head.dtype, device=device))
+            else:
+                self.caches.append(torch.zeros(num_slots, *mix.state_shape(), dtype=torch.float32, device=device))
+
+    # ---- forward ----
+    def forward(self, batch: RaggedBatch) -> torch.Tensor:
+        """Normed output [T, width] of every token of the batch."""
+        cfg, dtype, dev = self.cfg, self.head.dtype, self.head.device
+        T, W, eps = batch.tokens.numel(), cfg.width, cfg.norm_eps
+        rows = lambda: torch.empty(T, W, dtype=dtype, device=dev)
+        both = torch.empty(T, 2 * W, dtype=dtype, device=dev) if cfg.loop is not None else None   # [stream | embedding]
+        x = embed_rows(batch.tokens, self.embed, cfg.embedding_scale, both[:, W:] if both is not None else None)
+        h = rows()
+        n_runs = len(self.runs)
+        opens_pass = lambda r: r < n_runs and self.runs[r][1] is not None and self.runs[r][0] == cfg.loop.start
+
+        def hand_over(r, update, y, post):
+            """Apply the stream update that ends run r - 1 and write what run ``r`` reads first."""
+            norm = self.layers[self.runs[r][0]].norm1 if r < n_runs else self.final_norm
+            first_of_pass = opens_pass(r)
+            residual_norm(update, x, y, post, eps, both[:, :W] if first_of_pass else h, None if first_of_pass else norm)
+            if self.layer_hook is not None and r > 0:
+                self.layer_hook(r - 1, x)
+            if first_of_pass:
+                residual_norm(REPLACE, x, linear_f32(both, self.loop_in), self.loop_step[self.runs[r][1]], eps, h, norm)
+
+        hand_over(0, KEEP, None, None)
+        for r, (i, _) in enumerate(self.runs):
+            layer = self.layers[i]
+            y = layer.mix(h, batch, self.caches[r])
+            post = layer.post1
+            if layer.mlp is not None:
+                residual_norm(ADD_NORMED, x, y, post, eps, h, layer.norm2)
+                y, post = layer.mlp(h), layer.post2
+            if layer.side is not None:
+                residual_norm(ADD_NORMED, x, y, post, eps, h)
+                y, post = layer.side(h, batch.tokens, self.side_embed), layer.side.norm
+            hand_over(r + 1, ADD_NORMED, y, post)
+        return h
+
+    def compute_logits(self, hidden: torch.Tensor, batch: RaggedBatch) -> torch.Tensor:
+        """float32 logits of the batch's wanted rows."""
+        return linear_f32(hidden.index_select(0, batch.logit_rows), self.head)

@@ -42,9 +42,13 @@ def chain_digests(token_ids, block_size: int) -> List[int]:
 
 class KVBlockPool:
 
-    def __init__(self, num_blocks: int, block_size: int):
+    def __init__(self, num_blocks: int, block_size: int, reuse_prefix: bool = True):
+        """``reuse_prefix=False``: no block is ever shared or taken up again -- for models whose layers keep more than
+        cache rows (a recurrent state is not in the blocks), and for prompts that are computed in portions (a sealed
+        block might not be filled yet)."""
         if num_blocks <= 0:
             raise ValueError("the KV cache needs at least one block")
+        self.reuse_prefix = reuse_prefix
         self.block_size = block_size
         self.num_blocks = num_blocks
         self.refs = np.zeros(num_blocks, dtype=np.int32)
@@ -126,7 +130,7 @@ class KVBlockPool:
         assert not seq.block_table
         bs = self.block_size
         tokens = seq.token_ids
-        names = chain_digests(tokens, bs)
+        names = chain_digests(tokens, bs) if self.reuse_prefix else []
         reuse = []
         for i, name in enumerate(names):
             b = self._lookup(name, tokens[i * bs:(i + 1) * bs])
@@ -172,9 +176,39 @@ class KVBlockPool:
         table = seq.block_table
         if fill == 1:
             table.append(int(self._claim(self._head, keep_name=False)))
-        elif fill == 0:
+        elif fill == 0 and self.reuse_prefix:
             last = table[-1]
             assert not self.sealed[last]
             parent = int(self.digest[table[-2]]) if len(table) > 1 else _NIL
             tokens = seq.token_ids[-self.block_size:]
             self._seal(last, block_digest(tokens, parent), tokens)
+
+    # ---- a running request has grown by a portion of any size ----
+    def can_extend(self, seq: Sequence) -> bool:
+        return self.num_free >= seq.num_blocks - len(seq.block_table)
+
+    def extend(self, seq: Sequence) -> None:
+        """Make the table cover all of the request's tokens; the blocks get no names."""
+        while len(seq.block_table) < seq.num_blocks:
+            seq.block_table.append(int(self._claim(self._head, keep_name=False)))
+
+
+class StateSlotPool:
+    """Slots for the recurrent state of running requests, one each.  A slot is handed out as it is: the first token of
+    a request (position 0) starts from a zero state whatever the slot holds."""
+
+    def __init__(self, num_slots: int):
+        self.free = list(range(num_slots - 1, -1, -1))
+
+    @property
+    def num_free(self) -> int:
+        return len(self.free)
+
+    def take(self, seq: Sequence) -> None:
+        assert seq.state_slot < 0
+        seq.state_slot = self.free.pop()
+
+    def give_back(self, seq: Sequence) -> None:
+        if seq.state_slot >= 0:
+            self.free.append(seq.state_slot)
+            seq.state_slot = -1

@@ -15,6 +15,7 @@ import torch.nn.functional as F
 from torch import nn
 
 from ..layers.layernorm import RMSNorm
+from ..layers.moe.fused_moe import reserve_workspace
 from ..layers.moe.mixtral_block import MixtralMoE, PostAttentionMoE
 from .config import ModelConfig
 
@@ -111,9 +112,14 @@ class MixtralAttention(nn.Module):
         self.q_size, self.kv_size = nh * d, nkv * d
         # q, k and v rows stacked in one weight, as the reference's QKVParallelLinear keeps them
         self.qkv_proj = nn.Linear(cfg.hidden_size, self.q_size + 2 * self.kv_size, bias=False, dtype=cfg.torch_dtype)
+        self.qkv_proj.weight.weight_loader = self.load_qkv
         self.o_proj = nn.Linear(self.q_size, cfg.hidden_size, bias=False, dtype=cfg.torch_dtype)
         self.rotary_emb = RotaryEmbedding(d, cfg.max_position_embeddings, cfg.rope_theta)
         self.attn = PagedAttention(nh, nkv, d)
+
+    def load_qkv(self, param: nn.Parameter, loaded_weight: torch.Tensor, shard_id: str) -> None:
+        begin = {"q": 0, "k": self.q_size, "v": self.q_size + self.kv_size}[shard_id]
+        param.data[begin:begin + (self.q_size if shard_id == "q" else self.kv_size)].copy_(loaded_weight)
 
     def forward(self, positions: torch.Tensor, hidden_states: torch.Tensor, ctx: BatchContext) -> torch.Tensor:
         q, k, v = self.qkv_proj(hidden_states).split([self.q_size, self.kv_size, self.kv_size], dim=-1)
@@ -169,6 +175,31 @@ class MixtralForCausalLM(nn.Module):
         self.model.layers = nn.ModuleList([MixtralDecoderLayer(cfg, fused_moe_tail) for _ in range(cfg.num_hidden_layers)])
         self.model.norm = RMSNorm(cfg.hidden_size, eps=cfg.rms_norm_eps)
         self.lm_head = nn.Linear(cfg.hidden_size, cfg.vocab_size, bias=False, dtype=cfg.torch_dtype)
+
+    # q, k and v of the checkpoint are rows of one matrix
+    packed_modules_mapping = {"q_proj": ("qkv_proj", "q"), "k_proj": ("qkv_proj", "k"), "v_proj": ("qkv_proj", "v")}
+
+    def reserve_workspace(self, device, max_tokens: int) -> None:
+        """One MoE workspace for the largest batch the planner can form: no layer call allocates afterwards."""
+        cfg = self.cfg
+        reserve_workspace(device, max_tokens, cfg.hidden_size, cfg.intermediate_size, cfg.num_local_experts,
+                          cfg.num_experts_per_tok)
+
+    def cache_bytes(self, block_size: int) -> Tuple[int, int]:
+        """(bytes of a cache block over all layers, bytes of a state slot)."""
+        cfg = self.cfg
+        return (2 * cfg.num_hidden_layers * block_size * cfg.num_key_value_heads * cfg.head_dim *
+                self.lm_head.weight.element_size(), 0)
+
+    def allocate_cache(self, num_blocks: int, block_size: int, num_slots: int, device) -> None:
+        """[2, layers, blocks, block_size, kv_heads, head_dim]"""
+        cfg = self.cfg
+        kv = torch.zeros(2, cfg.num_hidden_layers, num_blocks, block_size, cfg.num_key_value_heads, cfg.head_dim,
+                         dtype=cfg.torch_dtype, device=device)
+        for i, layer in enumerate(self.model.layers):
+            layer.self_attn.attn.k_cache = kv[0, i]
+            layer.self_attn.attn.v_cache = kv[1, i]
+            layer.self_attn.attn.kv_cache = kv[:, i]
 
     def forward(self, input_ids: torch.Tensor, positions: torch.Tensor, ctx: BatchContext) -> torch.Tensor:
         hidden_states, residual = self.model.embed_tokens(input_ids), None

@@ -1,13 +1,15 @@
-"""Owns the model and the KV cache of one GPU and turns a scheduled batch into one forward pass and one sampled
+"""Owns the model, the cache and the states of one GPU and turns a scheduled batch into one forward pass and one sampled
 token per sequence (counterpart of electrock_infer/engine/model_runner.py:92-236, single process: the reference's
 shared-memory fan-out to tensor-parallel ranks has nothing to do on one GPU)."""
-from typing import List
+from typing import List, Optional
 
 import torch
 
-from ..layers.moe.fused_moe import reserve_workspace
+from ..utils.loader import load_model
+from .batch import make_ragged
 from .config import EngineConfig
-from .model import BatchContext, MixtralForCausalLM, Sampler
+from .model import BatchContext, Sampler
+from .registry import build_model
 from .sequence import Sequence
 
 
@@ -17,37 +19,33 @@ class ModelRunner:
         self.config = config
         self.block_size = config.kvcache_block_size
         self.device = torch.device(config.device)
-        cfg = config.model
         torch.cuda.set_device(self.device)
         with torch.device(self.device):
-            self.model = MixtralForCausalLM(cfg, fused_moe_tail=config.fused_moe_tail)
-        self.model.init_random_weights(config.seed)
+            self.model = build_model(config)
+        if config.model_dir is not None:
+            load_model(self.model, config.model_dir, device=str(self.device))
+        else:
+            self.model.init_random_weights(config.seed)
         self.sampler = Sampler()
-        # one MoE workspace for the largest batch the planner can form: no layer call allocates afterwards
-        reserve_workspace(self.device, config.max_num_batched_tokens, cfg.hidden_size, cfg.intermediate_size,
-                          cfg.num_local_experts, cfg.num_experts_per_tok)
+        self.ragged = getattr(self.model, "ragged_batches", False)
+        if hasattr(self.model, "reserve_workspace"):
+            self.model.reserve_workspace(self.device, config.max_num_batched_tokens)
         self.allocate_kv_cache()
 
     def allocate_kv_cache(self) -> None:
-        """[2, layers, blocks, block_size, kv_heads, head_dim]; the block count comes from the configuration or from
-        the device memory left under gpu_memory_utilization (model_runner.py:92-110)."""
-        config, cfg = self.config, self.config.model
-        block_bytes = 2 * cfg.num_hidden_layers * self.block_size * cfg.num_key_value_heads * cfg.head_dim * \
-            torch.empty((), dtype=cfg.torch_dtype).element_size()
+        """The model's cache for as many blocks as configured, or as fit into the device memory left under
+        gpu_memory_utilization (model_runner.py:92-110) behind the state slots."""
+        config = self.config
+        block_bytes, slot_bytes = self.model.cache_bytes(self.block_size)
         if config.num_kvcache_blocks <= 0:
             free, total = torch.cuda.mem_get_info(self.device)
-            budget = int(total * config.gpu_memory_utilization) - (total - free)
+            budget = int(total * config.gpu_memory_utilization) - (total - free) - slot_bytes * config.num_state_slots
             if budget < block_bytes:
                 raise RuntimeError("no device memory left for the KV cache")
             # what max_num_seqs sequences of max_model_len tokens can ever use is enough
             most = config.max_num_seqs * (-(-config.max_model_len // self.block_size))
-            config.num_kvcache_blocks = min(budget // block_bytes, most)
-        self.kv_cache = torch.zeros(2, cfg.num_hidden_layers, config.num_kvcache_blocks, self.block_size,
-                                    cfg.num_key_value_heads, cfg.head_dim, dtype=cfg.torch_dtype, device=self.device)
-        for i, layer in enumerate(self.model.model.layers):
-            layer.self_attn.attn.k_cache = self.kv_cache[0, i]
-            layer.self_attn.attn.v_cache = self.kv_cache[1, i]
-            layer.self_attn.attn.kv_cache = self.kv_cache[:, i]
+            config.num_kvcache_blocks = min(budget // block_bytes, most) if block_bytes else most
+        self.model.allocate_cache(config.num_kvcache_blocks, self.block_size, config.num_state_slots, self.device)
 
     # ---- batch preparation ----
     def _to_device(self, values, dtype) -> torch.Tensor:
@@ -57,18 +55,24 @@ class ModelRunner:
         width = max(len(s.block_table) for s in seqs)
         return self._to_device([s.block_table + [0] * (width - len(s.block_table)) for s in seqs], torch.int64)
 
+    def prepare_ragged(self, seqs: List[Sequence], rows: Optional[List[int]] = None):
+        """The planned portions of any batch, for models that take RaggedBatch; ``rows``: batch rows whose logits are
+        wanted (default: the last one of every sequence)."""
+        if any(not 0 <= s.state_slot < self.config.num_state_slots for s in seqs) and self.config.num_state_slots > 0:
+            raise ValueError("a sequence of this model needs a state slot")
+        return make_ragged(seqs, self.block_size, self.model.GLA_CHUNK, self.device, rows)
+
     def prepare_prefill(self, seqs: List[Sequence]):
-        """Feed the tokens behind every sequence's cached prefix; their cache slots follow from the block table."""
+        """Feed every sequence's planned portion behind its computed tokens; the cache slots follow from the block
+        table."""
         input_ids, positions, slots, q_lens, k_lens, last = [], [], [], [], [], []
         for seq in seqs:
-            n, cached = len(seq), seq.num_cached_tokens
-            if cached == n:          # everything was found in the prefix cache: still feed the last token
-                cached -= 1
-            input_ids.extend(seq[cached:])
-            positions.extend(range(cached, n))
-            q_lens.append(n - cached)
+            start, n = seq.num_computed_tokens, seq.num_computed_tokens + seq.num_scheduled_tokens
+            input_ids.extend(seq[start:n])
+            positions.extend(range(start, n))
+            q_lens.append(n - start)
             k_lens.append(n)
-            for pos in range(cached, n):
+            for pos in range(start, n):
                 slots.append(seq.block_table[pos // self.block_size] * self.block_size + pos % self.block_size)
             last.append(len(input_ids) - 1)
         need_tables = any(k != q for q, k in zip(q_lens, k_lens))
@@ -94,9 +98,28 @@ class ModelRunner:
     def run_model(self, input_ids, positions, ctx: BatchContext) -> torch.Tensor:
         return self.model.compute_logits(self.model(input_ids, positions, ctx), ctx)
 
+    @torch.inference_mode()
+    def run_ragged(self, seqs: List[Sequence], rows: Optional[List[int]] = None) -> torch.Tensor:
+        """Logits [wanted, vocab] of one forward pass over the planned portions."""
+        batch = self.prepare_ragged(seqs, rows)
+        return self.model.compute_logits(self.model(batch), batch)
+
+    def logits(self, seqs: List[Sequence], is_prefill: bool) -> torch.Tensor:
+        """Logits behind the last fed token of every sequence."""
+        if self.ragged:
+            return self.run_ragged(seqs)
+        return self.run_model(*(self.prepare_prefill(seqs) if is_prefill else self.prepare_decode(seqs)))
+
+    def portion_logits(self, seqs: List[Sequence], rows: List[int]) -> torch.Tensor:
+        """Logits of chosen rows of the planned portions (rows count through the batch)."""
+        if self.ragged:
+            return self.run_ragged(seqs, rows)
+        input_ids, positions, ctx = self.prepare_prefill(seqs)
+        ctx.last_token_index = self._to_device(rows, torch.int64)
+        return self.run_model(input_ids, positions, ctx)
+
     def run(self, seqs: List[Sequence], is_prefill: bool, return_logits: bool = False):
-        input_ids, positions, ctx = self.prepare_prefill(seqs) if is_prefill else self.prepare_decode(seqs)
         temperatures = self._to_device([s.temperature for s in seqs], torch.float32)
-        logits = self.run_model(input_ids, positions, ctx)
+        logits = self.logits(seqs, is_prefill)
         token_ids = self.sampler(logits, temperatures).tolist()
         return (token_ids, logits) if return_logits else token_ids

@@ -26,7 +26,11 @@ class Sequence:
         self.token_ids = list(token_ids)
         self.num_prompt_tokens = len(self.token_ids)
         self.num_cached_tokens = 0
+        self.num_computed_tokens = 0         # leading tokens whose cache rows (and state) exist
+        self.num_scheduled_tokens = 0        # tokens behind those that the planned step feeds
+        self.prefilling = False              # admitted, and not yet computed up to its newest token
         self.block_table = []
+        self.state_slot = -1                 # recurrent-state slot, for models that have one
         self.temperature = sampling_params.temperature
         self.max_tokens = sampling_params.max_tokens
         self.ignore_eos = sampling_params.ignore_eos

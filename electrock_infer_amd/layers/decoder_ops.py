@@ -1,0 +1,105 @@
+"""Row operations of a decoder whose residual stream is float32 (libelectrock_decoder.so), and the two matrix products
+around them.  Every function takes and returns GPU tensors; there is no other path."""
+import ctypes
+from typing import Optional
+
+import torch
+import torch.nn.functional as F
+
+from .. import _lib
+
+
+def _ptr(t: Optional[torch.Tensor]) -> Optional[int]:
+    return None if t is None else t.data_ptr()
+
+
+def linear_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """x @ weight^T with the float32 accumulators as the result, for sums that stay float32."""
+    if x.dtype == torch.float32:
+        return F.linear(x, weight)
+    return torch.mm(x, weight.t(), out_dtype=torch.float32)
+
+
+def embed_rows(tokens: torch.Tensor, table: torch.Tensor, scale: float, copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """float32 rows table[tokens] * scale; ``copy`` (rows may be strided) receives them in the table's type."""
+    T, W = tokens.numel(), table.shape[1]
+    x = torch.empty(T, W, dtype=torch.float32, device=table.device)
+    code = _lib.load_decoder().ed_embed(tokens.data_ptr(), table.data_ptr(), float(scale), x.data_ptr(), _ptr(copy),
+                                        copy.stride(0) if copy is not None else 0, T, W, _lib.dtype_code(table.dtype),
+                                        _lib.current_stream(table.device))
+    _lib.check_decoder(code, "embed_rows")
+    return x
+
+
+KEEP, ADD_NORMED, REPLACE = 0, 1, 2
+
+
+def residual_norm(update: int, x: torch.Tensor, y: Optional[torch.Tensor], post_w: Optional[torch.Tensor], eps: float,
+                  out: Optional[torch.Tensor], next_w: Optional[torch.Tensor] = None) -> None:
+    """Update the stream ``x`` in place (KEEP; ADD_NORMED: x += y / rms(y) * post_w; REPLACE: x = y + post_w) and write
+    the next sublayer's input into ``out`` (rows may be strided): x / rms(x) * next_w, or x itself, in out's type."""
+    T, W = x.shape
+    dtype = out.dtype if out is not None else (y.dtype if y is not None else x.dtype)
+    code = _lib.load_decoder().ed_residual_norm(
+        update, x.data_ptr(), _ptr(y), _lib.dtype_code(y.dtype if y is not None else dtype), _ptr(post_w), _ptr(next_w),
+        _ptr(out), out.stride(0) if out is not None else 0, T, W, float(eps), _lib.dtype_code(dtype),
+        _lib.current_stream(x.device))
+    _lib.check_decoder(code, "residual_norm")
+
+
+def relu_squared_(u: torch.Tensor) -> torch.Tensor:
+    code = _lib.load_decoder().ed_relu_squared(u.data_ptr(), u.numel(), _lib.dtype_code(u.dtype), _lib.current_stream(u.device))
+    _lib.check_decoder(code, "relu_squared")
+    return u
+
+
+def token_gate_(g: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, column0: int) -> torch.Tensor:
+    """g = gelu_tanh(g) * table[tokens, column0 : column0 + dim] in place."""
+    T, dim = g.shape
+    code = _lib.load_decoder().ed_token_gate(g.data_ptr(), tokens.data_ptr(), table.data_ptr(), table.stride(0), column0, T,
+                                             dim, _lib.dtype_code(g.dtype), _lib.current_stream(g.device))
+    _lib.check_decoder(code, "token_gate")
+    return g
+
+
+def pad_k(w: torch.Tensor) -> torch.Tensor:
+    """[heads, N, K] with K zero-padded to a multiple of 32: the operand form of ``head_gemm``."""
+    return F.pad(w, (0, -w.shape[-1] % 32)).contiguous()
+
+
+def head_gemm(a: torch.Tensor, a_row: int, a_head: int, b: torch.Tensor, K: int, out: torch.Tensor, out_row: int,
+              out_head: int, T: int) -> None:
+    """out[t, h, n] = sum_k a[t, h, k] b[h, n, k] (strides in elements; ``b`` from ``pad_k``)."""
+    heads, N, _ = b.shape
+    code = _lib.load_decoder().ed_head_gemm(a.data_ptr(), a_row, a_head, b.data_ptr(), out.data_ptr(), out_row, out_head, T,
+                                            heads, N, K, _lib.dtype_code(b.dtype), _lib.current_stream(b.device))
+    _lib.check_decoder(code, "head_gemm")
+
+
+class StackedLinear(torch.nn.Module):
+    """Several projections of one input as a single matrix: ``sections`` name -> rows, every section starting at a
+    multiple of eight rows (zeros between), so that vector loads of a section's outputs are aligned."""
+
+    def __init__(self, width: int, sections, dtype):
+        super().__init__()
+        self.offset, self.rows, at = {}, dict(sections), 0
+        for name, rows in self.rows.items():
+            self.offset[name] = at
+            at += (rows + 7) // 8 * 8
+        self.out_rows = at
+        self.weight = torch.nn.Parameter(torch.zeros(at, width, dtype=dtype), requires_grad=False)
+        self.weight.weight_loader = self.load_section
+
+    def load_section(self, param, loaded: torch.Tensor, name: str) -> None:
+        if loaded.shape != (self.rows[name], param.shape[1]):
+            raise ValueError(f"projection '{name}' is {tuple(loaded.shape)}, expected {(self.rows[name], param.shape[1])}")
+        param.data[self.offset[name]:self.offset[name] + self.rows[name]].copy_(loaded)
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return F.linear(x, self.weight)
+
+    def section_ptr(self, out: torch.Tensor, name: str) -> int:
+        return out.data_ptr() + self.offset[name] * out.element_size()
+
+
+byref = ctypes.byref

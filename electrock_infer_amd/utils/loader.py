@@ -8,6 +8,10 @@ to the ``weight_loader`` of the parameter it belongs to --
   stacked ``...experts.w13_weight`` / ``w2_weight`` through ``FusedMoE.weight_loader(param, tensor, shard, e)``,
 * everything else is copied by the parameter's own ``weight_loader`` or ``default_weight_loader``.
 
+A model with a naming of its own answers ``checkpoint_target(name) -> (parameter, shard id or None) | None`` instead; if
+it lists its ``expected_tensors()``, ``strict=True`` also raises for those that the files lack.  ``finish_loading()``,
+where a model has it, is called at the end (derived forms of the weights).
+
 ``strict=False`` skips tensors the model has no parameter for (a model made of the MoE block alone against a
 full checkpoint); the reference raises there, and so does ``strict=True``.
 """
@@ -40,14 +44,35 @@ def _find(model: nn.Module, name: str, strict: bool):
         return None
 
 
+def _load_named(model: nn.Module, target, name: str, file, strict: bool) -> bool:
+    param = _find(model, target[0], strict) if target is not None else None
+    if param is None:
+        if strict:
+            raise KeyError(f"the model has no parameter for '{name}'")
+        return False
+    tensor = file.get_tensor(name)
+    if target[1] is not None:
+        param.weight_loader(param, tensor, target[1])
+    elif tensor.shape != param.shape:
+        raise ValueError(f"'{name}' is {tuple(tensor.shape)}, expected {tuple(param.shape)}")
+    else:
+        getattr(param, "weight_loader", default_weight_loader)(param, tensor)
+    return True
+
+
 def load_model(model: nn.Module, path: str, rank: int = 0, device: str = "cpu", strict: bool = True) -> List[str]:
     """Load every ``*.safetensors`` file under ``path`` into ``model``; returns the names that were loaded."""
     packed = getattr(model, "packed_modules_mapping", {})
     experts = getattr(model, "experts_modules_mapping", EXPERTS_MODULES_MAPPING)
+    target_of = getattr(model, "checkpoint_target", None)
     loaded: List[str] = []
     for file in sorted(glob(os.path.join(path, "*.safetensors"))):
         with safe_open(file, "pt", device) as f:
             for weight_name in f.keys():
+                if target_of is not None:
+                    if _load_named(model, target_of(weight_name), weight_name, f, strict):
+                        loaded.append(weight_name)
+                    continue
                 done = False
                 for k in packed:
                     if k in weight_name:
@@ -74,4 +99,10 @@ def load_model(model: nn.Module, path: str, rank: int = 0, device: str = "cpu", 
                 if param is not None:
                     getattr(param, "weight_loader", default_weight_loader)(param, f.get_tensor(weight_name))
                     loaded.append(weight_name)
+    if strict and hasattr(model, "expected_tensors"):
+        missing = sorted(set(model.expected_tensors()) - set(loaded))
+        if missing:
+            raise KeyError(f"the checkpoint lacks {missing}")
+    if hasattr(model, "finish_loading"):
+        model.finish_loading()
     return loaded

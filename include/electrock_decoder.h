@@ -1,0 +1,121 @@
+/*
+ * electrock_decoder.h — C ABI of libelectrock_decoder.so (MI355X / gfx950): the kernels of decoders whose residual
+ * stream is float32 (row kernels), of gated linear attention and of latent attention over a paged cache.
+ *
+ * Same conventions as electrock_moe.h: raw DEVICE pointers, plain sizes, a HIP stream passed as void*; asynchronous,
+ * no allocation, no retained state; the device that owns the pointers is current.  Returns 0, an EM_ERR_* code (nothing
+ * was launched) or a hipError_t.
+ *
+ * Element types: EM_DTYPE_BF16 or EM_DTYPE_F32 is the compute type `dtype` of activations, weights and key cache.
+ * With EM_DTYPE_F32 every product is a float32 MFMA.  Pointers are aligned to 16 bytes unless said otherwise.
+ */
+#ifndef ELECTROCK_DECODER_H
+#define ELECTROCK_DECODER_H
+
+#include "electrock_moe.h"
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+int ed_version(void);
+
+/* x[t] = table[tokens[t]] * scale (float32 [T, W]); copy (may be null): the same, rounded to dtype, rows copy_stride
+ * elements apart. */
+int ed_embed(const int32_t* tokens, const void* table, double scale, float* x, void* copy, int64_t copy_stride,
+             int64_t T, int W, int dtype, void* stream);
+
+/* Update of the float32 stream x [T, W] by a sublayer's result y [T, W] (y_dtype), then the next sublayer's input:
+ *   update 0: x stays      1: x += y / sqrt(mean(y^2) + eps) * post_w      2: x = y + post_w (post_w may be null)
+ *   out (may be null): next_w ? x / sqrt(mean(x^2) + eps) * next_w : x, rounded to dtype, rows out_stride apart.
+ * post_w, next_w: float32 [W]. */
+int ed_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
+                     void* out, int64_t out_stride, int64_t T, int W, double eps, int dtype, void* stream);
+
+/* u = max(u, 0)^2, n elements in place. */
+int ed_relu_squared(void* u, int64_t n, int dtype, void* stream);
+
+/* g [T, dim] = gelu_tanh(g) * table[tokens[t]][column0 + c] in place; rows of the table are table_stride apart. */
+int ed_token_gate(void* g, const int32_t* tokens, const void* table, int64_t table_stride, int column0, int64_t T,
+                  int dim, int dtype, void* stream);
+
+/*
+ * Gated linear attention: S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T (q_scale q_t), alpha =
+ * sigmoid(a2 a1_t + bias)^(1/tau); o is RMS-normed per head with norm_w, multiplied by silu(g), rounded to dtype.
+ * q, k: head h at h * dim of a row; v, g: at h * vdim; all rows, and a1's, are `stride` elements apart.
+ * a2: [heads * dim, rank], rows a2_stride apart.  dim, vdim <= 256, rank <= 512.
+ * states: float32 [slots, heads, dim, vdim]; a sequence with starts[s] == 0 begins at zero, whatever its slot holds.
+ */
+typedef struct ed_gla_args {
+    const void *q, *k, *v, *g, *a1;
+    int64_t stride;
+    const void* a2;
+    const float* bias;
+    const float* norm_w;
+    void* out;                 /* [T, heads * vdim] */
+    const int32_t *slots;      /* [n_seqs] */
+    const int32_t *starts;     /* [n_seqs] position of the sequence's first token in this call */
+    float* states;
+    /* prompts only: */
+    float* log_decay;          /* [T, heads * dim] scratch */
+    const int32_t* chunks;     /* [n_chunks][4]: sequence, first row, tokens (<= chunk_tokens), unused */
+    const int32_t* seq_chunks; /* [n_seqs + 1] first chunk of every sequence; chunks of a sequence are consecutive */
+    float* chunk_states;       /* [n_chunks, heads, dim, vdim] scratch, null if every sequence has one chunk */
+    float* chunk_decay;        /* [n_chunks, heads, dim] scratch, null likewise */
+    int32_t n_seqs, n_chunks, chunk_tokens /* a multiple of 16 */;
+    int32_t heads, dim, vdim, rank, a2_stride, dtype;
+    float tau, q_scale, eps;
+} ed_gla_args;
+
+/* Portions of prompts: any number of tokens per sequence. */
+int ed_gla_prefill(const ed_gla_args* a, void* stream);
+/* One token per sequence: row s belongs to sequence s. */
+int ed_gla_step(const ed_gla_args* a, void* stream);
+
+/*
+ * Latent attention.  The cache holds, per token, round_up(rank, 8) elements of the normed latent and round_up(rot, 8) of
+ * the rotated key part (ed_latent_row_elems of them), zeros in the padding; key j of sequence s is row
+ * tables[s][j / block_size] * block_size + j % block_size.  rank <= 512, rot even and <= 128.
+ */
+typedef struct ed_latent_args {
+    void* q;                   /* rows q_stride apart, head h at h * (dim + rot): [dim plain, rot rotated] */
+    int64_t q_stride;
+    const void* down;          /* rows down_stride apart: [rank latent, rot key part] */
+    int64_t down_stride;
+    const float* latent_w;     /* [rank] */
+    const float* inv_freq;     /* [rot / 2] */
+    const int32_t* positions;  /* [T] */
+    const int32_t* cache_rows; /* [T] */
+    void* cache;
+    const void* q_latent;      /* [T, heads, round_up(rank, 8)] */
+    void* out;                 /* the same shape */
+    const float* sink;         /* [heads] */
+    const int32_t* q_begin;    /* [n_seqs + 1] first row of every sequence */
+    const int32_t* starts;     /* [n_seqs] position of that row's token */
+    const int32_t* tables;     /* [n_seqs, table_width] */
+    float* part_o;             /* [T * heads, splits, round_up(rank, 8)] scratch, unused if splits == 1 */
+    float* part_ml;            /* [T * heads, splits, 2] scratch */
+    int64_t T;
+    int32_t n_seqs, max_q, table_width, block_size, splits;
+    int32_t heads, dim, rot, rank, dtype;
+    float scale, eps;
+} ed_latent_args;
+
+int ed_latent_row_elems(int rank, int rot);
+/* Norm of the latent, rotation of the key part (both into the cache) and of q's rotated parts (in place). */
+int ed_latent_prepare(const ed_latent_args* a, void* stream);
+/* out = sum_j p_j c_j per row and head, p = softmax of (q_latent . c_j + q_rot . k_rot_j) * scale over the keys
+ * j <= position with exp(sink) added to the denominator; the keys of a row are shared out over `splits` workgroups. */
+int ed_latent_paged(const ed_latent_args* a, void* stream);
+/* out[t, h, n] = sum_k a[t, h, k] b[h][n][k]; b: [heads, N, round_up(K, 32)], zeros in the padding. */
+int ed_head_gemm(const void* a, int64_t a_row, int64_t a_head, const void* b, void* out, int64_t out_row,
+                 int64_t out_head, int64_t T, int heads, int N, int K, int dtype, void* stream);
+/* Cached rows of every sequence behind each other: out row k_begin[s] + j = key j of s, zeros from k_lens[s] on. */
+int ed_latent_gather(const void* cache, const int32_t* tables, int table_width, int block_size,
+                     const int32_t* k_begin, const int32_t* k_lens, int n_seqs, int max_k, int row_elems, void* out,
+                     int dtype, void* stream);
+
+#ifdef __cplusplus
+}
+#endif
+#endif
