@@ -1,6 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the Mixtral MoE layer on one MI355X.
 
+    python bench.py --model feguvik [--decoder-sizes 2048,4096]     (decoder models side by side; see decoder_rows)
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--tokens T] [--shape 8x7b|8x22b] [--mode MODE]
                     [--routing normal|zipf|two_experts|balanced] [--no-cpu] [--no-table] [--no-e2e] [--detail FILE]
 
@@ -103,6 +104,12 @@ def parse_args():
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="first run three device copies of 1 GiB (a plain copy kernel of known size that the "
                          "FETCH_SIZE / WRITE_SIZE counters of a rocprofv3 --pmc run are scaled by)")
+    ap.add_argument("--model", choices=["mixtral-moe-layer", "feguvik"], default="mixtral-moe-layer",
+                    help="feguvik: prefill and decode throughput of Feguvik models through the engine's runner, next to "
+                         "Mixtral models of equal size, instead of the MoE layer benchmark")
+    ap.add_argument("--decoder-sizes", default="2048,4096", help="widths of the --model feguvik rows")
+    ap.add_argument("--decoder-only", choices=["feguvik", "mixtral"], default=None,
+                    help="run one of the two models of the --model feguvik rows (profiling)")
     ap.add_argument("--detail", default=None, help="write the unabridged measurements to this JSON file")
     return ap.parse_args()
 
@@ -420,6 +427,91 @@ def compact_e2e(r):
             "decode_tok_s": sig(r["decode_tokens_per_s"]), "moe_share": sig(r["moe_share_of_gpu_time"], 3)}
 
 
+# ---- decoder models through the engine's runner ----
+def decoder_configs(width):
+    """A Feguvik model and a Mixtral model of equal width, heads, layer runs and active feed-forward flops (two of eight
+    experts with three matrices of I rows = a dense feed-forward with two matrices of 3 I rows)."""
+    from electrock_infer_amd.harness import FeguvikConfig, ModelConfig
+    from electrock_infer_amd.harness.feguvik import LayerSpec, LoopSpec
+    heads = width // 128
+    gla = LayerSpec("gla", {"heads": heads, "dim": 64, "vdim": 128, "tau": 16.0}, 3 * width, decay_rank=16)
+    mla = LayerSpec("latent_attention", {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512,
+                                         "rot": {"base": 10000.0, "dims": 64}, "scale": 192 ** -0.5}, 3 * width)
+    feg = FeguvikConfig(vocab_size=32000, width=width, layers=[gla, mla, gla, mla, gla, mla], norm_eps=1e-6,
+                        embedding_scale=1.0, side_dim=64, loop=LoopSpec(1, 3, 2))
+    mix = ModelConfig(vocab_size=32000, hidden_size=width, intermediate_size=width, num_hidden_layers=8,
+                      num_attention_heads=heads, num_key_value_heads=max(heads // 4, 1))
+    return {"feguvik": feg, "mixtral": mix}
+
+
+def decoder_rows(torch, name, cfg, width, steps, warmup):
+    """Prefill: one step over whole prompts.  Decode: steps of one token per sequence behind a 1024-token context, as the
+    engine runs them (batch preparation, forward pass, greedy sampling, token back on the host)."""
+    from random import Random
+    from electrock_infer_amd.harness import LLMEngine, SamplingParams
+    engine = LLMEngine(cfg, max_model_len=8704, max_num_seqs=64, max_num_batched_tokens=65536 if width <= 2048 else 32768,
+                       num_kvcache_blocks=4096, reuse_prefix=False)
+    rnd, rows = Random(0), []
+    sp = SamplingParams(temperature=0.0, max_tokens=100000, ignore_eos=True)
+
+    def prefill(lens):
+        for n in lens:
+            engine.add_request([rnd.randrange(32000) for _ in range(n)], sp)
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        _, fed = engine.step()
+        dt = time.perf_counter() - t0
+        assert fed == sum(lens)
+        return dt
+
+    def drop():
+        for s in engine.planner.running:
+            engine.planner.release(s)
+        engine.planner.running = []
+
+    for lens in ([8192], [1024] * 8, [2048], [512]):
+        times = []
+        for _ in range(warmup + steps):
+            times.append(prefill(lens))
+            drop()
+        ms = 1e3 * sorted(times[warmup:])[steps // 2]
+        rows.append({"model": name, "width": width, "phase": "prefill", "seqs": len(lens), "tokens": sum(lens), "ms": sig(ms),
+                     "tok_s": sig(sum(lens) / ms * 1e3)})
+    for batch in (1, 16, 64):
+        for _ in range(0, batch, 16):
+            prefill([1024] * min(batch, 16))
+        times = []
+        for _ in range(4 * (warmup + steps)):
+            t0 = time.perf_counter()
+            engine.step()
+            times.append(time.perf_counter() - t0)
+        ms = 1e3 * sorted(times[4 * warmup:])[2 * steps]
+        rows.append({"model": name, "width": width, "phase": "decode", "seqs": batch, "tokens": batch, "ms": sig(ms),
+                     "tok_s": sig(batch / ms * 1e3)})
+        drop()
+    del engine
+    from electrock_infer_amd.layers.moe.fused_moe import release_workspaces
+    release_workspaces()
+    torch.cuda.empty_cache()
+    return rows
+
+
+def decoder_bench(torch, args):
+    rows = []
+    for width in [int(w) for w in args.decoder_sizes.split(",")]:
+        for name, cfg in decoder_configs(width).items():
+            if args.decoder_only in (None, name):
+                rows += decoder_rows(torch, name, cfg, width, min(args.steps, 10), min(args.warmup, 3))
+                print(f"[decoder] {name} width {width} done", file=sys.stderr, flush=True)
+    head = rows[0]
+    print(json.dumps({"metric": f"{head['model']} prefill tokens/s", "value": head["tok_s"], "unit": "tokens/s", "n_gpus": 1,
+                      "steps": min(args.steps, 10), "warmup": min(args.warmup, 3), "ms_per_step": head["ms"],
+                      "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+                      "config": {"model": f"{head['model']} width {head['width']}, 8 layer runs, random weights",
+                                 "global_batch": head["seqs"], "seq_len": head["tokens"] // head["seqs"], "parallelism": "1"},
+                      "rows": rows}, separators=(",", ":")))
+
+
 def main():
     global OPERANDS
     args = parse_args()
@@ -434,6 +526,8 @@ def main():
         print("bench.py needs a GPU", file=sys.stderr)
         sys.exit(1)
     from electrock_infer_amd import _lib
+    if args.model == "feguvik":
+        return decoder_bench(torch, args)
     _lib.load()
     dev = torch.device("cuda:0")
     torch.cuda.set_device(dev)

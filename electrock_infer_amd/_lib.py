@@ -47,6 +47,7 @@ EXPORTED_SYMBOLS = (
 DECODER_SYMBOLS = (
     "ed_version", "ed_embed", "ed_residual_norm", "ed_relu_squared", "ed_token_gate", "ed_gla_prefill", "ed_gla_step",
     "ed_latent_row_elems", "ed_latent_prepare", "ed_latent_paged", "ed_head_gemm", "ed_latent_gather",
+    "ed_latent_prompt_supported", "ed_latent_prompt",
 )
 
 
@@ -70,6 +71,15 @@ class LatentArgs(ctypes.Structure):
                 [(n, ctypes.c_int32) for n in ("n_seqs", "max_q", "table_width", "block_size", "splits", "heads", "dim",
                                                "rot", "rank", "dtype")] +
                 [(n, ctypes.c_float) for n in ("scale", "eps")])
+
+
+class LatentPromptArgs(ctypes.Structure):
+    """Mirror of struct ed_latent_prompt_args."""
+    _fields_ = ([(n, t) for name in ("q", "k", "k_rot", "vt") for n, t in
+                 ((name, ctypes.c_void_p), (("v" if name == "vt" else name) + "_stride", ctypes.c_int64))] +
+                [(n, ctypes.c_void_p) for n in ("out", "sink", "q_begin", "starts", "k_begin")] +
+                [(n, ctypes.c_int32) for n in ("n_seqs", "max_q", "heads", "dim", "rot", "vdim")] +
+                [("scale", ctypes.c_float)])
 
 
 class MoeLayout(ctypes.Structure):
@@ -167,6 +177,8 @@ def load_decoder() -> ctypes.CDLL:
         "ed_latent_prepare": [ctypes.POINTER(LatentArgs), vp],
         "ed_latent_paged": [ctypes.POINTER(LatentArgs), vp],
         "ed_head_gemm": [vp, i64, i64, vp, vp, i64, i64, i64, i32, i32, i32, i32, vp],
+        "ed_latent_prompt_supported": [i32, i32, i32],
+        "ed_latent_prompt": [ctypes.POINTER(LatentPromptArgs), vp],
         "ed_latent_gather": [vp, vp, i32, i32, vp, vp, i32, i32, i32, vp, i32, vp],
     }
     for name, argtypes in signatures.items():

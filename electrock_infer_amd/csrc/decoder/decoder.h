@@ -82,4 +82,23 @@ int launch_head_gemm(const void* a, int64_t a_row, int64_t a_head, const void* b
 int launch_latent_gather(const void* cache, const int32_t* tables, int table_width, int block_size, const int32_t* k_begin,
                          const int32_t* k_lens, int n_seqs, int max_k, int row_elems, void* out, int dtype, hipStream_t s);
 
+// ---- latent_prompt.hip ----
+struct LatentPromptProblem {
+    const uint16_t* q;       // rotated already
+    int64_t q_stride;
+    const uint16_t* k;       // [keys, heads * dim], sequence s from row k_begin[s]
+    int64_t k_stride;
+    const uint16_t* k_rot;
+    int64_t k_rot_stride;
+    const uint16_t* vt;      // [heads * vdim, keys]
+    int64_t v_stride;
+    uint16_t* out;           // [T, heads * vdim]
+    const float* sink;
+    const int32_t *q_begin, *starts, *k_begin;
+    int heads, dim, rot, vdim;
+    float scale;
+};
+bool latent_prompt_supported(int dim, int rot, int vdim);
+int launch_latent_prompt(const LatentPromptProblem& p, int n_seqs, int max_q, hipStream_t s);
+
 }  // namespace em

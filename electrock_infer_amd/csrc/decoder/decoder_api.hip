@@ -173,4 +173,29 @@ int ed_latent_gather(const void* cache, const int32_t* tables, int table_width, 
                                 as_stream(stream));
 }
 
+int ed_latent_prompt_supported(int dim, int rot, int vdim) { return latent_prompt_supported(dim, rot, vdim) ? 1 : 0; }
+
+int ed_latent_prompt(const ed_latent_prompt_args* a, void* stream) {
+    if (!a) return EM_ERR_NULL_POINTER;
+    if (a->n_seqs < 0 || a->n_seqs > kMaxSeqs || a->max_q < 0 || a->max_q > kMaxRows || a->heads <= 0 || !(a->scale > 0.0f)) return EM_ERR_BAD_SHAPE;
+    if (!latent_prompt_supported(a->dim, a->rot, a->vdim) || a->q_stride % 8 != 0 || a->k_stride % 8 != 0 ||
+        a->k_rot_stride % 8 != 0 || a->v_stride % 8 != 0 || a->max_q > 128 * 65535)
+        return EM_ERR_UNSUPPORTED;
+    if (a->n_seqs == 0 || a->max_q == 0) return 0;
+    if (!a->q || !a->k || (a->rot > 0 && !a->k_rot) || !a->vt || !a->out || !a->sink || !a->q_begin || !a->starts || !a->k_begin)
+        return EM_ERR_NULL_POINTER;
+    if (!aligned16(a->q) || !aligned16(a->k) || !aligned16(a->k_rot) || !aligned16(a->vt) || !aligned16(a->out)) return EM_ERR_ALIGNMENT;
+    LatentPromptProblem p;
+    p.q = static_cast<const uint16_t*>(a->q); p.q_stride = a->q_stride;
+    p.k = static_cast<const uint16_t*>(a->k); p.k_stride = a->k_stride;
+    p.k_rot = static_cast<const uint16_t*>(a->k_rot); p.k_rot_stride = a->k_rot_stride;
+    p.vt = static_cast<const uint16_t*>(a->vt); p.v_stride = a->v_stride;
+    p.out = static_cast<uint16_t*>(a->out);
+    p.sink = a->sink;
+    p.q_begin = a->q_begin; p.starts = a->starts; p.k_begin = a->k_begin;
+    p.heads = a->heads; p.dim = a->dim; p.rot = a->rot; p.vdim = a->vdim;
+    p.scale = a->scale;
+    return launch_latent_prompt(p, a->n_seqs, a->max_q, as_stream(stream));
+}
+
 }  // extern "C"

@@ -17,8 +17,7 @@ class RaggedBatch:
     table_width: int
     n_chunks: int
     chunk_tokens: int
-    starts_host: List[int]          # position of every portion's first token
-    counts_host: List[int]
+    padded_keys: int                # all contexts behind each other, each padded to a multiple of 64
     tokens: torch.Tensor            # [T]
     positions: torch.Tensor         # [T]
     cache_rows: torch.Tensor        # [T] row of the paged cache that takes the token
@@ -28,6 +27,8 @@ class RaggedBatch:
     tables: torch.Tensor            # [n_seqs, table_width]
     chunks: torch.Tensor            # [n_chunks, 4] pieces of portions of at most chunk_tokens: sequence, row, tokens, 0
     seq_chunks: torch.Tensor        # [n_seqs + 1]
+    k_lens: torch.Tensor            # [n_seqs] context length, this step's tokens included
+    k_begin: torch.Tensor           # [n_seqs + 1] first of a sequence's padded keys
     logit_rows: torch.Tensor        # rows whose logits are wanted
 
 
@@ -51,6 +52,9 @@ def make_ragged(seqs: List[Sequence], block_size: int, chunk_tokens: int, device
     starts = [s.num_computed_tokens for s in seqs]
     counts = [s.num_scheduled_tokens for s in seqs]
     contexts = [a + n for a, n in zip(starts, counts)]
+    k_begin = [0]
+    for c in contexts:
+        k_begin.append(k_begin[-1] + -(-c // 64) * 64)
     width = max(-(-c // block_size) for c in contexts)
     tables = []
     for s, c in zip(seqs, contexts):
@@ -59,7 +63,7 @@ def make_ragged(seqs: List[Sequence], block_size: int, chunk_tokens: int, device
     wanted = last if rows is None else rows
     parts = {"tokens": tokens, "positions": positions, "cache_rows": cache_rows, "q_begin": q_begin, "starts": starts,
              "state_slots": [s.state_slot for s in seqs], "tables": tables, "chunks": chunks, "seq_chunks": seq_chunks,
-             "logit_rows": wanted}
+             "k_lens": contexts, "k_begin": k_begin, "logit_rows": wanted}
     flat, at = [], {}
     for name, values in parts.items():
         flat += [0] * (-len(flat) % 4)                  # 16-byte aligned views
@@ -71,4 +75,4 @@ def make_ragged(seqs: List[Sequence], block_size: int, chunk_tokens: int, device
     view["tables"] = view["tables"].view(len(seqs), width)
     view["chunks"] = view["chunks"].view(-1, 4)
     return RaggedBatch(n_seqs=len(seqs), max_q=max(counts), max_context=max(contexts), table_width=width,
-                       n_chunks=len(chunks) // 4, chunk_tokens=chunk_tokens, starts_host=starts, counts_host=counts, **view)
+                       n_chunks=len(chunks) // 4, chunk_tokens=chunk_tokens, padded_keys=k_begin[-1], **view)

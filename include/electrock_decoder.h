@@ -115,6 +115,31 @@ int ed_latent_gather(const void* cache, const int32_t* tables, int table_width, 
                      const int32_t* k_begin, const int32_t* k_lens, int n_seqs, int max_k, int row_elems, void* out,
                      int dtype, void* stream);
 
+/*
+ * Latent attention of long portions with the keys and values written out (bf16 only): k [keys, heads * dim], the
+ * transposed values vt [heads * vdim, keys] and the rotated key part k_rot, all for the whole context of every sequence,
+ * sequence s from key k_begin[s].  Every k_begin is a multiple of 64 and the rows (columns of vt) from a sequence's last
+ * key to the next multiple of 64 exist and are finite.  q is rotated already.  ed_latent_prompt_supported: which sizes.
+ */
+typedef struct ed_latent_prompt_args {
+    const void* q;             /* rows q_stride apart, head h at h * (dim + rot) */
+    int64_t q_stride;
+    const void* k;
+    int64_t k_stride;
+    const void* k_rot;
+    int64_t k_rot_stride;
+    const void* vt;
+    int64_t v_stride;
+    void* out;                 /* [T, heads * vdim] */
+    const float* sink;         /* [heads] */
+    const int32_t *q_begin, *starts, *k_begin; /* [n_seqs + 1], [n_seqs], [n_seqs] */
+    int32_t n_seqs, max_q, heads, dim, rot, vdim;
+    float scale;               /* > 0 */
+} ed_latent_prompt_args;
+
+int ed_latent_prompt_supported(int dim, int rot, int vdim);
+int ed_latent_prompt(const ed_latent_prompt_args* a, void* stream);
+
 #ifdef __cplusplus
 }
 #endif
