@@ -73,6 +73,7 @@ struct LatentProblem {
 };
 __host__ __device__ constexpr int latent_pitch(int rank) { return (rank + 7) / 8 * 8; }
 __host__ __device__ constexpr int latent_row_elems(int rank, int rot) { return latent_pitch(rank) + (rot + 7) / 8 * 8; }
+constexpr int kLatentMaxSplits = 256;
 bool latent_supported(int heads, int dim, int rot, int rank);
 int launch_latent_prepare(const LatentProblem& p, int64_t T, hipStream_t s);
 int launch_latent_paged(const LatentProblem& p, int n_seqs, int max_q, int splits, float* part_o, float* part_ml,

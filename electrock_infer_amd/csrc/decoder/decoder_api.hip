@@ -35,7 +35,7 @@ int check_gla(const ed_gla_args* a) {
     if (!a->q || !a->k || !a->v || !a->g || !a->a1 || !a->a2 || !a->bias || !a->norm_w || !a->out || !a->slots ||
         !a->starts || !a->states)
         return EM_ERR_NULL_POINTER;
-    if (!aligned16(a->states) || !aligned16(a->chunk_states)) return EM_ERR_ALIGNMENT;
+    if (!aligned16(a->states) || !aligned16(a->chunk_states) || !aligned16(a->a2)) return EM_ERR_ALIGNMENT;
     return 0;
 }
 
@@ -140,7 +140,7 @@ int ed_latent_prepare(const ed_latent_args* a, void* stream) {
 int ed_latent_paged(const ed_latent_args* a, void* stream) {
     const int rc = check_latent(a);
     if (rc != 0 || a->T == 0) return rc;
-    if (a->n_seqs <= 0 || a->n_seqs > kMaxSeqs || a->max_q <= 0 || a->max_q > a->T || a->splits < 1 || a->splits > 65535 ||
+    if (a->n_seqs <= 0 || a->n_seqs > kMaxSeqs || a->max_q <= 0 || a->max_q > a->T || a->splits < 1 || a->splits > kLatentMaxSplits ||
         a->block_size <= 0 || a->table_width <= 0)
         return EM_ERR_BAD_SHAPE;
     if (!a->q || !a->q_latent || !a->cache || !a->out || !a->sink || !a->q_begin || !a->starts || !a->tables) return EM_ERR_NULL_POINTER;

@@ -10,30 +10,37 @@
 // MFMA leaves its result; the same registers, as they are, are the second operand of the float32 16x16x4 MFMA.  One
 // workgroup is one (chunk, head), one wave a v tile.  Everything that reaches the state is float32: the operands are
 // products of the bf16 projections with float32 decays, and no exponent is positive except in the block's own 16 x 16
-// scores, where exp(-bl_s) is used as a factor only while the whole block decays by less than e^-kFactorLimit.
+// scores, where exp(-bl_s) is used as a factor only while the whole block decays by less than 2^-kFactorLimit.  (The
+// logarithms are kept to base 2.)
 // With more than one chunk in a sequence the chunks run in parallel: a first pass leaves every chunk's own contribution
 // to the state and its total decay, a scan over the chunks turns these into the states in front of them, and the
 // output pass starts from there.
 //
 // Decoding.  One workgroup per (sequence, head) streams the state once: decay, update, read-out, norm and gate.
+#include <type_traits>
+
 #include "decoder.h"
 
 namespace em {
 namespace {
 
 constexpr int kBlock = 16;
-constexpr float kFactorLimit = 40.0f;
+constexpr float kFactorLimit = 58.0f;  // log2
+constexpr float kLog2e = 1.4426950408889634f;
 constexpr int kPitchA = 20;   // floats between the rows of a 16 x 16 LDS matrix (16-byte reads of 4 columns)
 
+__device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
+// with the hardware's exponential and reciprocal, 1 ulp each
+__device__ __forceinline__ float silu_fast(float g) { return g * __builtin_amdgcn_rcpf(1.0f + exp2_fast(-g * kLog2e)); }
 __device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
 
-// bl [T, C]: per channel (C = heads * dim) the running sum of log alpha inside every block of 16 tokens.
+// bl [T, C]: per channel (C = heads * dim) the running sum of log2 alpha inside every block of 16 tokens.
 template <typename Elem>
 __global__ __launch_bounds__(256) void gla_decay_kernel(const typename Elem::storage* __restrict__ a1, int64_t a1_stride,
                                                         const typename Elem::storage* __restrict__ a2, int rank, int a2_stride,
                                                         const float* __restrict__ bias, float inv_tau,
                                                         const int4* __restrict__ chunks, float* __restrict__ bl, int C) {
-    extern __shared__ float lds_a1[];  // [16][rank]
+    extern __shared__ __attribute__((aligned(16))) float lds_a1[];  // [16][rank]
     const int4 ch = chunks[blockIdx.x];
     const int first = blockIdx.y * kBlock;
     if (first >= ch.z) return;
@@ -51,15 +58,28 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const typename Elem::sto
 #pragma unroll
     for (int t = 0; t < kBlock; ++t) z[t] = b;
     const typename Elem::storage* w = a2 + static_cast<int64_t>(c) * a2_stride;
-    for (int j = 0; j < rank; ++j) {
-        const float wj = Elem::load(w[j]);
+    if (rank % 4 == 0 && a2_stride % 4 == 0) {
+        for (int j = 0; j < rank; j += 4) {
+            typename Elem::storage ws[4];
+            __builtin_memcpy(ws, __builtin_assume_aligned(w + j, sizeof(ws)), sizeof(ws));
 #pragma unroll
-        for (int t = 0; t < kBlock; ++t) z[t] = fmaf(wj, lds_a1[t * rank + j], z[t]);
+            for (int t = 0; t < kBlock; ++t) {
+                const f32x4_t a = *reinterpret_cast<const f32x4_t*>(lds_a1 + t * rank + j);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) z[t] = fmaf(Elem::load(ws[i]), a[i], z[t]);
+            }
+        }
+    } else {
+        for (int j = 0; j < rank; ++j) {
+            const float wj = Elem::load(w[j]);
+#pragma unroll
+            for (int t = 0; t < kBlock; ++t) z[t] = fmaf(wj, lds_a1[t * rank + j], z[t]);
+        }
     }
     float sum = 0.0f;
 #pragma unroll
     for (int t = 0; t < kBlock; ++t) {
-        sum += log_sigmoid(z[t]) * inv_tau;
+        sum += log_sigmoid(z[t]) * (inv_tau * kLog2e);
         if (t < n) bl[(row0 + t) * C + c] = sum;
     }
 }
@@ -76,13 +96,24 @@ struct GlaArgs {
     const int32_t* starts;      // position of every sequence's first token in this step; 0: the state is zero
     float* states;              // [slots, heads, dim, vdim]
     float* chunk_states;        // [chunks, heads, dim, vdim]; null: one chunk per sequence, straight from / to the slots
-    float* chunk_decay;         // [chunks, heads, dim] sum of log alpha
+    float* chunk_decay;         // [chunks, heads, dim] sum of log2 alpha
     int heads, dim, vdim;
     float q_scale, eps;
 };
 
-template <typename Elem, int NDT, bool OUTPUT>
-__global__ __launch_bounds__(1024) void gla_chunk_kernel(GlaArgs p) {
+// What a thread of the chunk kernels loads for one block, ahead of its use: PAIRS pairs of neighbouring channels of q, k
+// and bl, and four rows of this lane's v and g columns.
+template <int PAIRS>
+struct BlockRegs {
+    uint32_t q[PAIRS], k[PAIRS];
+    f32x2_t b[PAIRS], tot[PAIRS];
+    uint16_t v[4], g[4];
+};
+
+// PAIRS > 0 (bf16, even dim, at most PAIRS * 2 * threads channel values per block, at most 512 threads): the next
+// block's operands are in flight while this one is computed.  PAIRS == 0: any size, element by element.
+template <typename Elem, int NDT, bool OUTPUT, int PAIRS>
+__global__ __launch_bounds__(PAIRS > 0 ? 512 : 1024, PAIRS > 0 && NDT > 4 ? 2 : 4) void gla_chunk_kernel(GlaArgs p) {
     typedef typename Elem::storage S;
     constexpr int D = NDT * 16;
     constexpr int DP = D + 4;
@@ -123,39 +154,91 @@ __global__ __launch_bounds__(1024) void gla_chunk_kernel(GlaArgs p) {
             st[dt][r] = (!from_zero && v_ok && d < dim) ? mine[static_cast<int64_t>(d) * vdim + vc] : 0.0f;
         }
     const float nw = (OUTPUT && v_ok) ? p.norm_w[vc] : 0.0f;
+    const float inv_vdim = 1.0f / static_cast<float>(vdim);
     if (!OUTPUT)
         for (int d = tid; d < dim; d += blockDim.x) Bl[d] = 0.0f;  // here: the chunk's decay so far
+
+    BlockRegs<PAIRS ? PAIRS : 1> regs;
+    auto fetch = [&](int first) {
+        const int n = min(kBlock, ch.z - first);
+        const int64_t row0 = static_cast<int64_t>(ch.y) + first;
+#pragma unroll
+        for (int i = 0; i < PAIRS; ++i) {
+            const int e = (tid + i * static_cast<int>(blockDim.x)) * 2, t = e / D, d = e - t * D;
+            regs.q[i] = regs.k[i] = 0;
+            regs.b[i] = regs.tot[i] = f32x2_t{0.0f, 0.0f};
+            if (t < kBlock && d < dim) {
+                regs.tot[i] = *reinterpret_cast<const f32x2_t*>(p.bl + (row0 + n - 1) * C + h * dim + d);
+                regs.b[i] = regs.tot[i];
+                if (t < n) {
+                    regs.b[i] = *reinterpret_cast<const f32x2_t*>(p.bl + (row0 + t) * C + h * dim + d);
+                    regs.k[i] = *reinterpret_cast<const uint32_t*>(kg + (row0 + t) * p.stride + d);
+                    if (OUTPUT) regs.q[i] = *reinterpret_cast<const uint32_t*>(qg + (row0 + t) * p.stride + d);
+                }
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int t = lq * 4 + r;
+            const bool ok = v_ok && t < n;
+            regs.v[r] = ok ? static_cast<uint16_t>(vg[(row0 + t) * p.stride + vc]) : 0;
+            if (OUTPUT) regs.g[r] = ok ? static_cast<uint16_t>(gg[(row0 + t) * p.stride + vc]) : 0;
+        }
+    };
+    if (PAIRS > 0) fetch(0);
 
     for (int first = 0; first < ch.z; first += kBlock) {
         const int n = min(kBlock, ch.z - first);
         const int64_t row0 = static_cast<int64_t>(ch.y) + first;
         // ---- operands of the block ----
         bool factor_ok = true;
-        for (int i = tid; i < kBlock * D; i += blockDim.x) {
-            const int t = i / D, d = i - t * D;
-            float q = 0.0f, k = 0.0f, b = 0.0f, tot = 0.0f;
-            if (d < dim) {
-                tot = p.bl[(row0 + n - 1) * C + h * dim + d];
-                b = tot;
-                if (t < n) {
-                    b = p.bl[(row0 + t) * C + h * dim + d];
-                    k = Elem::load(kg[(row0 + t) * p.stride + d]);
-                    if (OUTPUT) q = Elem::load(qg[(row0 + t) * p.stride + d]) * p.q_scale;
-                }
-            }
-            if (t == 0) Et[d] = expf(tot);
-            Kt[d * kPitchA + t] = k * expf(tot - b);
+        auto place = [&](int t, int d, float q, float k, float b, float tot) {
+            if (t == 0) Et[d] = exp2_fast(tot);
+            Kt[d * kPitchA + t] = k * exp2_fast(tot - b);
             if (OUTPUT) {
-                Qp[t * DP + d] = q * expf(b);
-                Kn[t * DP + d] = k * expf(fminf(-b, kFactorLimit));
+                Qp[t * DP + d] = q * exp2_fast(b);
+                Kn[t * DP + d] = k * exp2_fast(fminf(-b, kFactorLimit));
                 factor_ok = factor_ok && tot > -kFactorLimit;
             }
-        }
-        float v[4];
+        };
+        float v[4], gate[4];
+        if (PAIRS > 0) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int t = lq * 4 + r;
-            v[r] = (v_ok && t < n) ? Elem::load(vg[(row0 + t) * p.stride + vc]) : 0.0f;
+            for (int i = 0; i < PAIRS; ++i) {
+                const int e = (tid + i * static_cast<int>(blockDim.x)) * 2, t = e / D, d = e - t * D;
+                if (t < kBlock) {
+                    place(t, d, bf16_lo(regs.q[i]) * p.q_scale, bf16_lo(regs.k[i]), regs.b[i][0], regs.tot[i][0]);
+                    place(t, d + 1, bf16_hi(regs.q[i]) * p.q_scale, bf16_hi(regs.k[i]), regs.b[i][1], regs.tot[i][1]);
+                }
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                v[r] = bf16_bits_to_f32(regs.v[r]);
+                gate[r] = OUTPUT ? bf16_bits_to_f32(regs.g[r]) : 0.0f;
+            }
+            if (first + kBlock < ch.z) fetch(first + kBlock);
+        } else {
+            for (int i = tid; i < kBlock * D; i += blockDim.x) {
+                const int t = i / D, d = i - t * D;
+                float q = 0.0f, k = 0.0f, b = 0.0f, tot = 0.0f;
+                if (d < dim) {
+                    tot = p.bl[(row0 + n - 1) * C + h * dim + d];
+                    b = tot;
+                    if (t < n) {
+                        b = p.bl[(row0 + t) * C + h * dim + d];
+                        k = Elem::load(kg[(row0 + t) * p.stride + d]);
+                        if (OUTPUT) q = Elem::load(qg[(row0 + t) * p.stride + d]) * p.q_scale;
+                    }
+                }
+                place(t, d, q, k, b, tot);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int t = lq * 4 + r;
+                const bool ok = v_ok && t < n;
+                v[r] = ok ? Elem::load(vg[(row0 + t) * p.stride + vc]) : 0.0f;
+                gate[r] = OUTPUT && ok ? Elem::load(gg[(row0 + t) * p.stride + vc]) : 0.0f;
+            }
         }
         if (OUTPUT) {
             factor_ok = __syncthreads_and(factor_ok);
@@ -175,21 +258,26 @@ __global__ __launch_bounds__(1024) void gla_chunk_kernel(GlaArgs p) {
                     Bl[t * DP + d] = (d < dim && t < n) ? p.bl[(row0 + t) * C + h * dim + d] : 0.0f;
                 }
                 __syncthreads();
+#pragma unroll 1
                 for (int r = 0; r < 4; ++r) {
                     const int t = lq * 4 + r, s = l16;
-                    if (s > t || t >= n) continue;
-                    const S* qr = qg + (row0 + t) * p.stride;
-                    const S* kr = kg + (row0 + s) * p.stride;
                     float sum = 0.0f;
-                    for (int d = wave; d < dim; d += waves)
-                        sum += Elem::load(qr[d]) * p.q_scale * Elem::load(kr[d]) * expf(Bl[t * DP + d] - Bl[s * DP + d]);
-                    a[r] = sum;
+                    if (s <= t && t < n) {
+                        const S* qr = qg + (row0 + t) * p.stride;
+                        const S* kr = kg + (row0 + s) * p.stride;
+                        for (int d = wave; d < dim; d += waves)
+                            sum += Elem::load(qr[d]) * p.q_scale * Elem::load(kr[d]) * exp2_fast(Bl[t * DP + d] - Bl[s * DP + d]);
+                    }
+                    a = f32x4_t{r == 0 ? sum : a[0], r == 1 ? sum : a[1], r == 2 ? sum : a[2], r == 3 ? sum : a[3]};
                 }
             }
+            // (waves beyond the channel tiles have nothing to add)
+            if (wave < NDT || !factor_ok) {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = lq * 4 + r;
-                Ap[(wave * kBlock + t) * kPitchA + l16] = l16 <= t ? a[r] : 0.0f;
+                for (int r = 0; r < 4; ++r) {
+                    const int t = lq * 4 + r;
+                    Ap[(wave * kBlock + t) * kPitchA + l16] = l16 <= t ? a[r] : 0.0f;
+                }
             }
         }
         __syncthreads();
@@ -203,7 +291,8 @@ __global__ __launch_bounds__(1024) void gla_chunk_kernel(GlaArgs p) {
                 for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[r], st[dt][r], o, 0, 0, 0);
             }
             f32x4_t a4 = {0.0f, 0.0f, 0.0f, 0.0f};
-            for (int w = 0; w < waves; ++w)
+            const int parts = factor_ok ? min(waves, NDT) : waves;
+            for (int w = 0; w < parts; ++w)
                 a4 += *reinterpret_cast<const f32x4_t*>(Ap + (w * kBlock + l16) * kPitchA + lq * 4);
 #pragma unroll
             for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(a4[r], v[r], o, 0, 0, 0);
@@ -231,15 +320,14 @@ __global__ __launch_bounds__(1024) void gla_chunk_kernel(GlaArgs p) {
         }
         __syncthreads();  // the block's LDS operands are no longer needed
         if (OUTPUT) {
+            f32x4_t ss = {0.0f, 0.0f, 0.0f, 0.0f};
+            for (int w = 0; w < waves; ++w) ss += *reinterpret_cast<const f32x4_t*>(Rs + w * kBlock + lq * 4);
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int t = lq * 4 + r;
-                float ss = 0.0f;
-                for (int w = 0; w < waves; ++w) ss += Rs[w * kBlock + t];
                 if (v_ok && t < n) {
-                    const float g = Elem::load(gg[(row0 + t) * p.stride + vc]);
-                    const float y = o[r] / sqrtf(ss / static_cast<float>(vdim) + p.eps) * nw;
-                    static_cast<S*>(p.out)[(row0 + t) * p.heads * vdim + h * vdim + vc] = Elem::store(y * silu(g));
+                    const float y = o[r] * __builtin_amdgcn_rsqf(ss[r] * inv_vdim + p.eps) * nw;
+                    static_cast<S*>(p.out)[(row0 + t) * p.heads * vdim + h * vdim + vc] = Elem::store(y * silu_fast(gate[r]));
                 }
             }
         }
@@ -284,7 +372,7 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaArgs p, const int32_t*
         for (int j = 0; j < kAhead; ++j)
             if (c + j < c1) {
                 cs[(c + j) * pitch] = state;
-                state = fmaf(expf(e[j]), state, u[j]);
+                state = fmaf(exp2_fast(e[j]), state, u[j]);
             }
     }
     *slot = state;
@@ -378,21 +466,29 @@ size_t chunk_lds_bytes(int ndt, int waves) {
     return sizeof(float) * (3 * kBlock * DP + D * kPitchA + D + waves * kBlock * kPitchA + waves * kBlock);
 }
 
-template <typename Elem, int NDT>
-int launch_chunks(const GlaArgs& p, int n_chunks, bool output, hipStream_t s) {
+template <typename Elem, int NDT, bool OUTPUT, int PAIRS>
+int launch_chunk_kernel(const GlaArgs& p, int n_chunks, hipStream_t s) {
     const int waves = static_cast<int>(ceil_div(p.vdim, 16));
     const dim3 grid(static_cast<unsigned>(n_chunks), static_cast<unsigned>(p.heads)), block(static_cast<unsigned>(waves * kWave));
     const size_t lds = chunk_lds_bytes(NDT, waves);
-    if (output) {
-        const int rc = allow_lds(reinterpret_cast<const void*>(gla_chunk_kernel<Elem, NDT, true>), lds);
-        if (rc != 0) return rc;
-        launch((gla_chunk_kernel<Elem, NDT, true>), grid, block, lds, s, p);
-    } else {
-        const int rc = allow_lds(reinterpret_cast<const void*>(gla_chunk_kernel<Elem, NDT, false>), lds);
-        if (rc != 0) return rc;
-        launch((gla_chunk_kernel<Elem, NDT, false>), grid, block, lds, s, p);
-    }
+    const int rc = allow_lds(reinterpret_cast<const void*>(gla_chunk_kernel<Elem, NDT, OUTPUT, PAIRS>), lds);
+    if (rc != 0) return rc;
+    launch((gla_chunk_kernel<Elem, NDT, OUTPUT, PAIRS>), grid, block, lds, s, p);
     return launch_status();
+}
+
+template <typename Elem, int NDT>
+int launch_chunks(const GlaArgs& p, int n_chunks, bool output, hipStream_t s) {
+    const int threads = static_cast<int>(ceil_div(p.vdim, 16)) * kWave;
+    const int pairs = static_cast<int>(ceil_div(kBlock * NDT * 16 / 2, threads));
+    if (std::is_same<Elem, BF16Elem>::value && p.dim % 2 == 0 && pairs <= 2 && threads <= 512) {
+        if (pairs == 1)
+            return output ? launch_chunk_kernel<BF16Elem, NDT, true, 1>(p, n_chunks, s)
+                          : launch_chunk_kernel<BF16Elem, NDT, false, 1>(p, n_chunks, s);
+        return output ? launch_chunk_kernel<BF16Elem, NDT, true, 2>(p, n_chunks, s)
+                      : launch_chunk_kernel<BF16Elem, NDT, false, 2>(p, n_chunks, s);
+    }
+    return output ? launch_chunk_kernel<Elem, NDT, true, 0>(p, n_chunks, s) : launch_chunk_kernel<Elem, NDT, false, 0>(p, n_chunks, s);
 }
 
 template <typename Elem>

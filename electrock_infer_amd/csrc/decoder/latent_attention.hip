@@ -78,22 +78,33 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const typename Elem::sto
     for (int m = 0; m < MT; ++m)
 #pragma unroll
         for (int n = 0; n < NT; ++n) acc[m][n] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
-    for (int k = lq * 8; k < KP; k += 32) {
-        typename M::frag fa[MT], fb[NT];
+    constexpr int kSteps = MT == 4 ? 2 : 4;  // k steps whose operands are in flight together
+    for (int k0 = 0; k0 < KP; k0 += 32 * kSteps) {
+        typename M::frag fa[kSteps][MT], fb[kSteps][NT];
 #pragma unroll
-        for (int m = 0; m < MT; ++m) {
-            const int64_t t = t0 + m * 16 + l16;
-            fa[m] = t < T ? load_frag<Elem>(a + t * a_row + h * a_head + k, K - k, vec) : M::zero();
+        for (int u = 0; u < kSteps; ++u) {
+            const int k = k0 + u * 32 + lq * 8;
+            if (k0 + u * 32 < KP) {
+#pragma unroll
+                for (int m = 0; m < MT; ++m) {
+                    const int64_t t = t0 + m * 16 + l16;
+                    fa[u][m] = t < T ? load_frag<Elem>(a + t * a_row + h * a_head + k, K - k, vec) : M::zero();
+                }
+#pragma unroll
+                for (int n = 0; n < NT; ++n) {
+                    const int col = n0 + n * 16 + l16;
+                    fb[u][n] = col < N ? M::load(bh + static_cast<int64_t>(col) * KP + k) : M::zero();
+                }
+            }
         }
 #pragma unroll
-        for (int n = 0; n < NT; ++n) {
-            const int col = n0 + n * 16 + l16;
-            fb[n] = col < N ? M::load(bh + static_cast<int64_t>(col) * KP + k) : M::zero();
-        }
+        for (int u = 0; u < kSteps; ++u)
+            if (k0 + u * 32 < KP) {
 #pragma unroll
-        for (int m = 0; m < MT; ++m)
+                for (int m = 0; m < MT; ++m)
 #pragma unroll
-            for (int n = 0; n < NT; ++n) acc[m][n] = M::mac(fa[m], fb[n], acc[m][n]);
+                    for (int n = 0; n < NT; ++n) acc[m][n] = M::mac(fa[u][m], fb[u][n], acc[m][n]);
+            }
     }
 #pragma unroll
     for (int m = 0; m < MT; ++m)
@@ -107,12 +118,40 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const typename Elem::sto
             }
 }
 
+// Rows row0 .. row0 + 7 of column col0 + l16 of an LDS matrix: the second operand's fragment of a matrix that lies with
+// its k dimension across rows.
+template <typename Elem>
+__device__ __forceinline__ typename Mma<Elem>::frag load_transposed(const typename Elem::storage* m, int pitch, int row0,
+                                                                    int col0, int l16);
+template <>
+__device__ __forceinline__ f32x8_t load_transposed<F32Elem>(const float* m, int pitch, int row0, int col0, int l16) {
+    f32x8_t f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f[i] = m[(row0 + i) * pitch + col0 + l16];
+    return f;
+}
+template <>
+__device__ __forceinline__ bf16x8_t load_transposed<BF16Elem>(const uint16_t* m, int pitch, int row0, int col0, int l16) {
+    // ds_read_b64_tr_b16: the 16 lanes of a group name the four-element pieces of a 4 x 16 block, row by row, and lane i
+    // receives column i of it
+    typedef short s16x4_t __attribute__((ext_vector_type(4)));
+    typedef __attribute__((address_space(3))) s16x4_t* lds_ptr;
+    const uint16_t* a = m + (row0 + (l16 >> 2)) * pitch + col0 + (l16 & 3) * 4;
+    const s16x4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)(a));
+    const s16x4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)(a + 4 * pitch));
+    bf16x8_t f;
+    __builtin_memcpy(&f, &lo, 8);
+    __builtin_memcpy(reinterpret_cast<char*>(&f) + 8, &hi, 8);
+    return f;
+}
+
 // ---- attention over the pages ----
 // A workgroup takes 16 (token, head) rows of one sequence, heads fastest, and one of `splits` ranges of their keys.
 // Per tile of 32 keys: the tile goes through registers into LDS (the next one is fetched while this one is used), the
 // four waves split the score product over key halves and channel halves, 16 threads per row keep the row's running
 // maximum and sum, and for the values (the latents again) each wave owns a quarter of the latent's columns.
 constexpr int kKeys = 32;
+constexpr int kMaxSplits = kLatentMaxSplits;
 
 template <typename Elem> struct LdsPad { static constexpr int n = 16 / sizeof(typename Elem::storage); };
 
@@ -143,12 +182,13 @@ __global__ __launch_bounds__(256) void latent_paged_kernel(LatentProblem p, int 
     S* Pm = Ks + kKeys * LP;                            // [16][PP]
     float* Sc = reinterpret_cast<float*>(Pm + 16 * PP); // [2][16][33]
     float* Al = Sc + 2 * 16 * 33;                       // [16]
+    int* Kr = reinterpret_cast<int*>(Al + 16);          // [2][32] cache row of every key of a tile, -1: no key
 
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lq = lane >> 4;
     const int pieces = row_elems / 8;                   // per key
 
     // queries: [latent | rotated], zeros behind; the same columns of the key rows
-    const bool q_vec = pitch_c % 8 == 0;
+    const bool rot_vec = p.rot % 8 == 0 && p.dim % 8 == 0 && p.q_stride % 8 == 0;
     for (int i = tid; i < 16 * (DK / 8); i += 256) {
         const int r = i / (DK / 8), c = (i - r * (DK / 8)) * 8;
         typename M::frag f = M::zero();
@@ -156,10 +196,10 @@ __global__ __launch_bounds__(256) void latent_paged_kernel(LatentProblem p, int 
             const int t = (r0 + r) / p.heads, h = (r0 + r) - t * p.heads;
             const int64_t row = q0 + t;
             if (c < pitch_c) {
-                f = load_frag<Elem>(static_cast<const S*>(p.q_latent) + (row * p.heads + h) * pitch_c + c, p.rank - c, q_vec);
+                f = load_frag<Elem>(static_cast<const S*>(p.q_latent) + (row * p.heads + h) * pitch_c + c, p.rank - c, true);
             } else if (c < row_elems) {
                 f = load_frag<Elem>(static_cast<const S*>(p.q) + row * p.q_stride + h * (p.dim + p.rot) + p.dim + (c - pitch_c),
-                                    p.rot - (c - pitch_c), false);
+                                    p.rot - (c - pitch_c), rot_vec);
             }
         }
         store_frag<Elem>(Qs + r * LP + c, f);
@@ -180,15 +220,19 @@ __global__ __launch_bounds__(256) void latent_paged_kernel(LatentProblem p, int 
     const int32_t* table = p.tables + static_cast<int64_t>(seq) * p.table_width;
     const S* cache = static_cast<const S*>(p.cache);
     typename M::frag fetched[kFetch];
+    auto find_rows = [&](int tile) {
+        if (tid < kKeys && tile < tile1) {
+            const int key = tile * kKeys + tid, blk = key / p.block_size;
+            Kr[(tile & 1) * kKeys + tid] = key < n_keys ? table[blk] * p.block_size + (key - blk * p.block_size) : -1;
+        }
+    };
     auto fetch = [&](int tile) {
 #pragma unroll
         for (int i = 0; i < kFetch; ++i) {
-            const int key = tile * kKeys + pk[i];
             fetched[i] = M::zero();
-            if (pk[i] < kKeys && key < n_keys) {
-                const int blk = key / p.block_size;
-                const int64_t row = static_cast<int64_t>(table[blk]) * p.block_size + (key - blk * p.block_size);
-                fetched[i] = M::load(cache + row * row_elems + pc[i]);
+            if (pk[i] < kKeys) {
+                const int row = Kr[(tile & 1) * kKeys + pk[i]];
+                if (row >= 0) fetched[i] = M::load(cache + static_cast<int64_t>(row) * row_elems + pc[i]);
             }
         }
     };
@@ -201,6 +245,9 @@ __global__ __launch_bounds__(256) void latent_paged_kernel(LatentProblem p, int 
     const int spos = start + min(r0 + srow, rows - 1) / p.heads;
     float m = -INFINITY, l = 0.0f;
 
+    find_rows(tile0);
+    find_rows(tile0 + 1);
+    __syncthreads();
     if (tile0 < tile1) fetch(tile0);
     for (int tile = tile0; tile < tile1; ++tile) {
         __syncthreads();   // the previous tile has been used (and, the first time, Qs is written)
@@ -209,6 +256,7 @@ __global__ __launch_bounds__(256) void latent_paged_kernel(LatentProblem p, int 
             if (pk[i] < kKeys) store_frag<Elem>(Ks + pk[i] * LP + pc[i], fetched[i]);
         if (tile + 1 < tile1) fetch(tile + 1);
         __syncthreads();
+        find_rows(tile + 2);     // into the half that this tile's rows leave; read behind the next barriers
         {
             f32x4_t s = {0.0f, 0.0f, 0.0f, 0.0f};
             const S* qp = Qs + l16 * LP + lq * 8;
@@ -253,12 +301,8 @@ __global__ __launch_bounds__(256) void latent_paged_kernel(LatentProblem p, int 
             for (int n = 0; n < NTW; ++n) {
                 const int c = (wave * NTW + n) * 16;
                 if (c < pitch_c) {
-                    typename M::frag fv;
-                    const S* vp = Ks + lq * 8 * LP + c + l16;
-#pragma unroll
-                    for (int i = 0; i < 8; ++i) M::set(fv, i, vp[i * LP]);
                     o[n] *= a4;
-                    o[n] = M::mac(fp, fv, o[n]);
+                    o[n] = M::mac(fp, load_transposed<Elem>(Ks, LP, lq * 8, c, l16), o[n]);
                 }
             }
         }
@@ -304,6 +348,8 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(const float* __rest
                                                              const float* __restrict__ part_ml,
                                                              const float* __restrict__ sink, int heads, int splits,
                                                              int pitch, int rank, typename Elem::storage* __restrict__ out) {
+    constexpr int kAhead = 8;
+    __shared__ float weight[kMaxSplits];
     const int64_t row = blockIdx.x;
     const float* ml = part_ml + row * splits * 2;
     const float sk = sink[row % heads];
@@ -311,13 +357,22 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(const float* __rest
     for (int s = 0; s < splits; ++s) top = fmaxf(top, ml[2 * s]);
     float den = expf(sk - top);
     for (int s = 0; s < splits; ++s) den += ml[2 * s + 1] * expf(ml[2 * s] - top);
-    for (int c = threadIdx.x; c < pitch; c += 128) {
-        float v = 0.0f;
-        if (c < rank) {
-            for (int s = 0; s < splits; ++s) v += part_o[(row * splits + s) * pitch + c] * expf(ml[2 * s] - top);
-            v /= den;
+    for (int s = threadIdx.x; s < splits; s += 128) weight[s] = expf(ml[2 * s] - top) / den;
+    __syncthreads();
+    for (int c = threadIdx.x * 4; c < pitch; c += 512) {   // pitch is a multiple of eight
+        const f32x4_t* src = reinterpret_cast<const f32x4_t*>(part_o + row * splits * pitch + c);
+        f32x4_t v = {0.0f, 0.0f, 0.0f, 0.0f};
+        for (int s0 = 0; s0 < splits; s0 += kAhead) {
+            f32x4_t x[kAhead];
+#pragma unroll
+            for (int j = 0; j < kAhead; ++j)
+                x[j] = s0 + j < splits ? src[static_cast<int64_t>(s0 + j) * pitch / 4] : f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+            for (int j = 0; j < kAhead; ++j)
+                if (s0 + j < splits) v += x[j] * weight[s0 + j];
         }
-        out[row * pitch + c] = Elem::store(v);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) out[row * pitch + c + j] = Elem::store(c + j < rank ? v[j] : 0.0f);
     }
 }
 
@@ -346,7 +401,7 @@ template <typename Elem, int NTW>
 int launch_paged(const LatentProblem& p, int n_seqs, int max_q, int splits, float* part_o, float* part_ml, hipStream_t s) {
     typedef typename Elem::storage S;
     const int DK = static_cast<int>(round_up(latent_row_elems(p.rank, p.rot), 32)), LP = DK + LdsPad<Elem>::n;
-    const size_t lds = sizeof(S) * (48 * LP + 16 * (kKeys + LdsPad<Elem>::n)) + sizeof(float) * (2 * 16 * 33 + 16);
+    const size_t lds = sizeof(S) * (48 * LP + 16 * (kKeys + LdsPad<Elem>::n)) + sizeof(float) * (2 * 16 * 33 + 16 + 2 * kKeys);
     const int rc = allow_lds(reinterpret_cast<const void*>(latent_paged_kernel<Elem, NTW>), lds);
     if (rc != 0) return rc;
     const dim3 grid(static_cast<unsigned>(ceil_div(static_cast<int64_t>(max_q) * p.heads, 16)), static_cast<unsigned>(n_seqs),
@@ -373,12 +428,18 @@ int head_gemm(const void* a, int64_t a_row, int64_t a_head, const void* b, void*
               int64_t T, int heads, int N, int K, hipStream_t s) {
     typedef typename Elem::storage S;
     const bool vec = a_row % 8 == 0 && a_head % 8 == 0 && reinterpret_cast<uintptr_t>(a) % (8 * sizeof(S)) == 0;
-    const int waves = static_cast<int>(ceil_div(N, 64)) < 4 ? static_cast<int>(ceil_div(N, 64)) : 4;
-    const int mt = T > 16 ? 4 : 1;
+    // as many rows per workgroup as leave the chip filled
+    const int64_t cols = ceil_div(N, 64);
+    const int mt = ceil_div(T, 64) * cols * heads >= 512 ? 4 : T > 16 && ceil_div(T, 32) * cols * heads >= 256 ? 2 : 1;
+    const int64_t wave_tiles = ceil_div(T, 16 * mt) * cols * heads;
+    const int waves = static_cast<int>(wave_tiles >= 1024 ? (cols < 4 ? cols : 4) : 1);
     const dim3 grid(static_cast<unsigned>(ceil_div(T, 16 * mt)), static_cast<unsigned>(ceil_div(N, waves * 64)),
                     static_cast<unsigned>(heads)), block(static_cast<unsigned>(waves * kWave));
     if (mt == 4)
         launch((head_gemm_kernel<Elem, 4>), grid, block, 0, s, static_cast<const S*>(a), a_row, a_head,
+               static_cast<const S*>(b), static_cast<S*>(out), o_row, o_head, T, N, K, vec);
+    else if (mt == 2)
+        launch((head_gemm_kernel<Elem, 2>), grid, block, 0, s, static_cast<const S*>(a), a_row, a_head,
                static_cast<const S*>(b), static_cast<S*>(out), o_row, o_head, T, N, K, vec);
     else
         launch((head_gemm_kernel<Elem, 1>), grid, block, 0, s, static_cast<const S*>(a), a_row, a_head,

@@ -105,7 +105,7 @@ int ed_latent_row_elems(int rank, int rot);
 /* Norm of the latent, rotation of the key part (both into the cache) and of q's rotated parts (in place). */
 int ed_latent_prepare(const ed_latent_args* a, void* stream);
 /* out = sum_j p_j c_j per row and head, p = softmax of (q_latent . c_j + q_rot . k_rot_j) * scale over the keys
- * j <= position with exp(sink) added to the denominator; the keys of a row are shared out over `splits` workgroups. */
+ * j <= position with exp(sink) added to the denominator; the keys of a row are shared out over `splits` (<= 256) workgroups. */
 int ed_latent_paged(const ed_latent_args* a, void* stream);
 /* out[t, h, n] = sum_k a[t, h, k] b[h][n][k]; b: [heads, N, round_up(K, 32)], zeros in the padding. */
 int ed_head_gemm(const void* a, int64_t a_row, int64_t a_head, const void* b, void* out, int64_t out_row,
