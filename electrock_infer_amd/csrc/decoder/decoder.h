@@ -25,8 +25,28 @@ int launch_embed(const int32_t* tokens, const void* table, float scale, float* x
 int launch_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
                          void* out, int64_t out_stride, int64_t T, int W, float eps, int dtype, hipStream_t s);
 int launch_relu_squared(void* u, int64_t n, int dtype, hipStream_t s);
-int launch_token_gate(void* g, const int32_t* tokens, const void* table, int64_t table_stride, int column0, int64_t T,
-                      int dim, int dtype, hipStream_t s);
+
+// ---- token_side.hip ----
+struct TokenSideProblem {
+    float* x;                // [T, W]
+    const uint16_t* y;       // [T, W]
+    const float *post_w, *side_norm, *next_w;
+    const uint16_t *gate, *proj;   // [dim, W], [W, dim]
+    const int32_t* tokens;
+    const uint16_t* table;
+    int64_t table_stride;
+    int column0;
+    uint16_t* out;
+    int64_t out_stride;
+    int64_t T;
+    int W, dim;
+    float eps;
+    int rows_per_group, g_offset, part_offset;  // set by the launcher
+};
+int launch_token_gate(const void* x, const void* gate, const int32_t* tokens, const void* table, int64_t table_stride,
+                      int column0, void* g, int64_t T, int W, int dim, int dtype, hipStream_t s);
+bool token_side_supported(int W, int dim);
+int launch_token_side(TokenSideProblem p, hipStream_t s);
 
 // ---- gla.hip ----
 struct GlaProblem {

@@ -100,13 +100,46 @@ int ed_relu_squared(void* u, int64_t n, int dtype, void* stream) {
     return launch_relu_squared(u, n, dtype, as_stream(stream));
 }
 
-int ed_token_gate(void* g, const int32_t* tokens, const void* table, int64_t table_stride, int column0, int64_t T,
-                  int dim, int dtype, void* stream) {
+int ed_token_gate(const void* x, const void* gate, const int32_t* tokens, const void* table, int64_t table_stride,
+                  int column0, void* g, int64_t T, int W, int dim, int dtype, void* stream) {
     if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
-    if (T < 0 || T > kMaxRows || dim <= 0 || column0 < 0 || column0 + static_cast<int64_t>(dim) > table_stride) return EM_ERR_BAD_SHAPE;
+    if (T < 0 || T > kMaxRows || W <= 0 || dim <= 0 || dim > 16 * 65535 || column0 < 0 ||
+        column0 + static_cast<int64_t>(dim) > table_stride)
+        return EM_ERR_BAD_SHAPE;
     if (T == 0) return 0;
-    if (!g || !tokens || !table) return EM_ERR_NULL_POINTER;
-    return launch_token_gate(g, tokens, table, table_stride, column0, T, dim, dtype, as_stream(stream));
+    if (!x || !gate || !tokens || !table || !g) return EM_ERR_NULL_POINTER;
+    if (!aligned16(x) || !aligned16(gate)) return EM_ERR_ALIGNMENT;
+    return launch_token_gate(x, gate, tokens, table, table_stride, column0, g, T, W, dim, dtype, as_stream(stream));
+}
+
+int ed_token_side_supported(int W, int dim) { return token_side_supported(W, dim) ? 1 : 0; }
+
+int ed_token_side(float* x, const void* y, const float* post_w, const void* gate, const void* proj, const int32_t* tokens,
+                  const void* table, int64_t table_stride, int column0, const float* side_norm, const float* next_w, void* out,
+                  int64_t out_stride, int64_t T, int W, int dim, double eps, void* stream) {
+    if (T < 0 || T > kMaxRows || column0 < 0 || column0 + static_cast<int64_t>(dim) > table_stride || out_stride < W) return EM_ERR_BAD_SHAPE;
+    if (!token_side_supported(W, dim) || out_stride % 4 != 0) return EM_ERR_UNSUPPORTED;
+    if (T == 0) return 0;
+    if (!x || !y || !post_w || !gate || !proj || !tokens || !table || !side_norm || !out) return EM_ERR_NULL_POINTER;
+    if (!aligned16(x) || !aligned16(y) || !aligned16(post_w) || !aligned16(gate) || !aligned16(proj) || !aligned16(side_norm) ||
+        !aligned16(next_w) || !aligned16(out))
+        return EM_ERR_ALIGNMENT;
+    TokenSideProblem p{};
+    p.x = x;
+    p.y = static_cast<const uint16_t*>(y);
+    p.post_w = post_w; p.side_norm = side_norm; p.next_w = next_w;
+    p.gate = static_cast<const uint16_t*>(gate);
+    p.proj = static_cast<const uint16_t*>(proj);
+    p.tokens = tokens;
+    p.table = static_cast<const uint16_t*>(table);
+    p.table_stride = table_stride;
+    p.column0 = column0;
+    p.out = static_cast<uint16_t*>(out);
+    p.out_stride = out_stride;
+    p.T = T;
+    p.W = W; p.dim = dim;
+    p.eps = static_cast<float>(eps);
+    return launch_token_side(p, as_stream(stream));
 }
 
 int ed_gla_prefill(const ed_gla_args* a, void* stream) {

@@ -1,5 +1,5 @@
 // Row kernels of a decoder whose residual stream is float32: embedding, post-norm residual update fused with the next
-// layer's pre-norm, squared ReLU, and the gate of a per-layer token input.
+// layer's pre-norm, and squared ReLU.
 #include "decoder.h"
 
 namespace em {
@@ -155,20 +155,6 @@ __global__ __launch_bounds__(256) void relu_squared_kernel(typename Elem::storag
     RowIo<Elem, VEC>::store(u + i, v);
 }
 
-// g = gelu_tanh(g) * table[token][column0 ...] in place; g [T, dim]
-template <typename Elem>
-__global__ __launch_bounds__(256) void token_gate_kernel(typename Elem::storage* __restrict__ g,
-                                                         const int32_t* __restrict__ tokens,
-                                                         const typename Elem::storage* __restrict__ table,
-                                                         int64_t table_stride, int column0, int64_t n, int dim) {
-    const int64_t i = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
-    if (i >= n) return;
-    const int64_t t = i / dim;
-    const int c = static_cast<int>(i - t * dim);
-    const float e = Elem::load(table[static_cast<int64_t>(tokens[t]) * table_stride + column0 + c]);
-    g[i] = Elem::store(gelu_tanh(Elem::load(g[i])) * e);
-}
-
 template <typename Elem, typename YElem, int UPDATE, int VEC>
 int launch_residual(float* x, const void* y, const float* post_w, const float* next_w, void* out, int64_t out_stride,
                     int64_t T, int W, float eps, hipStream_t s) {
@@ -236,19 +222,6 @@ int launch_relu_squared(void* u, int64_t n, int dtype, hipStream_t s) {
         if (vec == 8) launch((relu_squared_kernel<F32Elem, 8>), grid, dim3(256), 0, s, static_cast<float*>(u), n);
         else launch((relu_squared_kernel<F32Elem, 1>), grid, dim3(256), 0, s, static_cast<float*>(u), n);
     }
-    return launch_status();
-}
-
-int launch_token_gate(void* g, const int32_t* tokens, const void* table, int64_t table_stride, int column0, int64_t T,
-                      int dim, int dtype, hipStream_t s) {
-    const int64_t n = T * dim;
-    const dim3 grid(static_cast<unsigned>(ceil_div(n, 256)));
-    if (dtype == EM_DTYPE_BF16)
-        launch((token_gate_kernel<BF16Elem>), grid, dim3(256), 0, s, static_cast<uint16_t*>(g), tokens,
-               static_cast<const uint16_t*>(table), table_stride, column0, n, dim);
-    else
-        launch((token_gate_kernel<F32Elem>), grid, dim3(256), 0, s, static_cast<float*>(g), tokens,
-               static_cast<const float*>(table), table_stride, column0, n, dim);
     return launch_status();
 }
 

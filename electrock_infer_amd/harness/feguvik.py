@@ -210,28 +210,29 @@ class FeguvikForCausalLM(nn.Module):
         n_runs = len(self.runs)
         opens_pass = lambda r: r < n_runs and self.runs[r][1] is not None and self.runs[r][0] == cfg.loop.start
 
-        def hand_over(r, update, y, post):
-            """Apply the stream update that ends run r - 1 and write what run ``r`` reads first."""
+        def open_run(r, update):
+            """``update(out, norm)`` changes the stream and writes x / rms(x) * norm, or x for None: what run ``r`` reads."""
             norm = self.layers[self.runs[r][0]].norm1 if r < n_runs else self.final_norm
-            first_of_pass = opens_pass(r)
-            residual_norm(update, x, y, post, eps, both[:, :W] if first_of_pass else h, None if first_of_pass else norm)
+            if not opens_pass(r):
+                update(h, norm)
+            else:
+                update(both[:, :W], None)
             if self.layer_hook is not None and r > 0:
                 self.layer_hook(r - 1, x)
-            if first_of_pass:
+            if opens_pass(r):
                 residual_norm(REPLACE, x, linear_f32(both, self.loop_in), self.loop_step[self.runs[r][1]], eps, h, norm)
 
-        hand_over(0, KEEP, None, None)
+        open_run(0, lambda out, norm: residual_norm(KEEP, x, None, None, eps, out, norm))
         for r, (i, _) in enumerate(self.runs):
             layer = self.layers[i]
-            y = layer.mix(h, batch, self.caches[r])
-            post = layer.post1
+            y, post = layer.mix(h, batch, self.caches[r]), layer.post1
             if layer.mlp is not None:
                 residual_norm(ADD_NORMED, x, y, post, eps, h, layer.norm2)
                 y, post = layer.mlp(h), layer.post2
             if layer.side is not None:
-                residual_norm(ADD_NORMED, x, y, post, eps, h)
-                y, post = layer.side(h, batch.tokens, self.side_embed), layer.side.norm
-            hand_over(r + 1, ADD_NORMED, y, post)
+                open_run(r + 1, lambda out, norm: layer.side.close_layer(x, y, post, batch.tokens, self.side_embed, eps, out, norm))
+            else:
+                open_run(r + 1, lambda out, norm: residual_norm(ADD_NORMED, x, y, post, eps, out, norm))
         return h
 
     def compute_logits(self, hidden: torch.Tensor, batch: RaggedBatch) -> torch.Tensor:

@@ -53,11 +53,12 @@ def relu_squared_(u: torch.Tensor) -> torch.Tensor:
     return u
 
 
-def token_gate_(g: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, column0: int) -> torch.Tensor:
-    """g = gelu_tanh(g) * table[tokens, column0 : column0 + dim] in place."""
-    T, dim = g.shape
-    code = _lib.load_decoder().ed_token_gate(g.data_ptr(), tokens.data_ptr(), table.data_ptr(), table.stride(0), column0, T,
-                                             dim, _lib.dtype_code(g.dtype), _lib.current_stream(g.device))
+def token_gate(x: torch.Tensor, gate: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, column0: int) -> torch.Tensor:
+    """gelu_tanh(x @ gate^T) * table[tokens, column0 : column0 + dim]"""
+    (T, W), dim = x.shape, gate.shape[0]
+    g = torch.empty(T, dim, dtype=x.dtype, device=x.device)
+    code = _lib.load_decoder().ed_token_gate(x.data_ptr(), gate.data_ptr(), tokens.data_ptr(), table.data_ptr(), table.stride(0),
+                                             column0, g.data_ptr(), T, W, dim, _lib.dtype_code(x.dtype), _lib.current_stream(x.device))
     _lib.check_decoder(code, "token_gate")
     return g
 

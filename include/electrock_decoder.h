@@ -35,9 +35,19 @@ int ed_residual_norm(int update, float* x, const void* y, int y_dtype, const flo
 /* u = max(u, 0)^2, n elements in place. */
 int ed_relu_squared(void* u, int64_t n, int dtype, void* stream);
 
-/* g [T, dim] = gelu_tanh(g) * table[tokens[t]][column0 + c] in place; rows of the table are table_stride apart. */
-int ed_token_gate(void* g, const int32_t* tokens, const void* table, int64_t table_stride, int column0, int64_t T,
-                  int dim, int dtype, void* stream);
+/* g [T, dim] = gelu_tanh(x gate^T) * table[tokens[t]][column0 + c]; x [T, W], gate [dim, W]. */
+int ed_token_gate(const void* x, const void* gate, const int32_t* tokens, const void* table, int64_t table_stride,
+                  int column0, void* g, int64_t T, int W, int dim, int dtype, void* stream);
+
+/* The end of a layer with a per-layer token input in one launch (bf16; W a multiple of 4, see
+ * ed_token_side_supported):
+ *   x += y / rms(y) * post_w;  g = gelu_tanh(gate x) * table[tokens[t]][column0 ...];  p = proj g;
+ *   x += p / rms(p) * side_norm;  out = next_w ? x / rms(x) * next_w : x, rounded to bf16.
+ * gate [dim, W], proj [W, dim]; rms(v) = sqrt(mean(v^2) + eps); norm weights float32. */
+int ed_token_side_supported(int W, int dim);
+int ed_token_side(float* x, const void* y, const float* post_w, const void* gate, const void* proj, const int32_t* tokens,
+                  const void* table, int64_t table_stride, int column0, const float* side_norm, const float* next_w, void* out,
+                  int64_t out_stride, int64_t T, int W, int dim, double eps, void* stream);
 
 /*
  * Gated linear attention: S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T (q_scale q_t), alpha =

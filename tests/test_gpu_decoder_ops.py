@@ -80,6 +80,35 @@ def test_feed_forward_and_token_side_input(dtype):
 
 
 @pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("T,W,dim", [(1, 92, 5), (9, 260, 64), (33, 256, 24), (530, 128, 100), (17, 2048, 64), (40, 1024, 160), (530, 384, 32), (20, 4092, 16), (19, 4096, 96), (3, 4100, 7)])
+def test_end_of_a_layer_with_token_side_input(T, W, dim, dtype):
+    """The one-launch form and the form in steps (float32, or a width that the first does not take)."""
+    announce(f"token side, end of layer T={T} W={W} dim={dim} {dtype}")
+    eps, vocab, layer = 1e-4, 13, 1
+    w = {"l1.side.gate": rand(dim, W, seed=4, scale=W ** -0.5), "l1.side.proj": rand(W, dim, seed=5), "side.embed": rand(vocab, 3 * dim, seed=7)}
+    w = {k: v.to(dtype).float() for k, v in w.items()}
+    w["l1.side.norm"] = rand(W, seed=6)
+    x, y, post, nxt = rand(T, W, seed=1), rand(T, W, seed=2).to(dtype).float(), rand(W, seed=3), rand(W, seed=8)
+    toks = torch.arange(T) * 5 % vocab
+    ref = x + F.rms_norm(y, post, eps)
+    ref = ref + F.token_side_input(ref, toks, w, layer, dim, eps)
+    side = TokenSideInput(W, dim, layer * dim, dtype).to(DEV)
+    side.gate.data.copy_(w["l1.side.gate"]), side.proj.data.copy_(w["l1.side.proj"]), side.norm.data.copy_(w["l1.side.norm"])
+    both = torch.full((T, 2 * W), 5.0, dtype=dtype, device=DEV)
+    for next_w, out, one_launch in ((nxt, torch.empty(T, W, dtype=dtype, device=DEV), 1), (None, both[:, :W], 1),
+                                    (nxt, torch.empty(T, W, dtype=dtype, device=DEV), 10 ** 9)):
+        xg, side.ONE_LAUNCH_ROWS = to(x), one_launch
+        side.close_layer(xg, to(y, dtype), to(post), toks.int().to(DEV), to(w["side.embed"], dtype), eps, out,
+                         None if next_w is None else to(next_w))
+        close(xg, ref, dtype)
+        close(out, ref if next_w is None else F.rms_norm(ref, next_w, eps), dtype)
+        # no row is worse than the others: the rows of a tile do not mix
+        rows = (xg.cpu() - ref).pow(2).mean(-1).sqrt()
+        assert float(rows.max()) < (1e-4 if dtype == F32 else 5e-2)
+    assert bool((both[:, W:] == 5).all())
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
 @pytest.mark.parametrize("T,H,N,K", [(1, 3, 5, 7), (16, 2, 64, 32), (17, 5, 70, 33), (90, 1, 300, 130)])
 def test_head_gemm(T, H, N, K, dtype):
     announce(f"head gemm {T} {H} {N} {K} {dtype}")
