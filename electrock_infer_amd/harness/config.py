@@ -65,6 +65,7 @@ class EngineConfig:
     fused_moe_tail: bool = True         # post-attention norm + gate + router + experts in one library call
     prefill_portion: int = 0            # compute prompts in portions of at most so many tokens (0: whole)
     reuse_prefix: bool = True           # share cache blocks of equal prefixes (off for models with a recurrent state)
+    decode_graphs: bool = True          # record decode steps as HIP graphs, for models that take ragged batches
     num_state_slots: int = 0            # recurrent-state slots; set to max_num_seqs for models that have such a state
 
     def __post_init__(self):

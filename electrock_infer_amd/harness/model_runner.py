@@ -8,6 +8,7 @@ import torch
 from ..utils.loader import load_model
 from .batch import make_ragged
 from .config import EngineConfig
+from .decode_graph import DecodeGraphs
 from .model import BatchContext, Sampler
 from .registry import build_model
 from .sequence import Sequence
@@ -27,7 +28,7 @@ class ModelRunner:
         else:
             self.model.init_random_weights(config.seed)
         self.sampler = Sampler()
-        self.ragged = getattr(self.model, "ragged_batches", False)
+        self.ragged = getattr(self.model, "ragged_batches", False)      # takes RaggedBatch (batch.py)
         if hasattr(self.model, "reserve_workspace"):
             self.model.reserve_workspace(self.device, config.max_num_batched_tokens)
         self.allocate_kv_cache()
@@ -45,7 +46,10 @@ class ModelRunner:
             # what max_num_seqs sequences of max_model_len tokens can ever use is enough
             most = config.max_num_seqs * (-(-config.max_model_len // self.block_size))
             config.num_kvcache_blocks = min(budget // block_bytes, most) if block_bytes else most
-        self.model.allocate_cache(config.num_kvcache_blocks, self.block_size, config.num_state_slots, self.device)
+        # (one block and one slot more than the planner hands out, for the unused rows of padded decode steps)
+        extra = 1 if self.ragged else 0
+        self.model.allocate_cache(config.num_kvcache_blocks + extra, self.block_size, config.num_state_slots + extra, self.device)
+        self.graphs = DecodeGraphs(self) if self.ragged and config.decode_graphs else None
 
     # ---- batch preparation ----
     def _to_device(self, values, dtype) -> torch.Tensor:
@@ -55,11 +59,14 @@ class ModelRunner:
         width = max(len(s.block_table) for s in seqs)
         return self._to_device([s.block_table + [0] * (width - len(s.block_table)) for s in seqs], torch.int64)
 
+    def check_slots(self, seqs: List[Sequence]) -> None:
+        if self.config.num_state_slots > 0 and any(not 0 <= s.state_slot < self.config.num_state_slots for s in seqs):
+            raise ValueError("a sequence of this model needs a state slot")
+
     def prepare_ragged(self, seqs: List[Sequence], rows: Optional[List[int]] = None):
         """The planned portions of any batch, for models that take RaggedBatch; ``rows``: batch rows whose logits are
         wanted (default: the last one of every sequence)."""
-        if any(not 0 <= s.state_slot < self.config.num_state_slots for s in seqs) and self.config.num_state_slots > 0:
-            raise ValueError("a sequence of this model needs a state slot")
+        self.check_slots(seqs)
         return make_ragged(seqs, self.block_size, self.model.GLA_CHUNK, self.device, rows)
 
     def prepare_prefill(self, seqs: List[Sequence]):
@@ -100,7 +107,12 @@ class ModelRunner:
 
     @torch.inference_mode()
     def run_ragged(self, seqs: List[Sequence], rows: Optional[List[int]] = None) -> torch.Tensor:
-        """Logits [wanted, vocab] of one forward pass over the planned portions."""
+        """Logits [wanted, vocab] of one forward pass over the planned portions.  A decode step is the replay of a
+        recorded graph where one can be had (the result is overwritten by the next replay of that graph)."""
+        if self.graphs is not None and rows is None and all(s.num_scheduled_tokens == 1 for s in seqs):
+            logits = self.graphs.run(seqs)
+            if logits is not None:
+                return logits
         batch = self.prepare_ragged(seqs, rows)
         return self.model.compute_logits(self.model(batch), batch)
 
@@ -119,7 +131,10 @@ class ModelRunner:
         return self.run_model(input_ids, positions, ctx)
 
     def run(self, seqs: List[Sequence], is_prefill: bool, return_logits: bool = False):
-        temperatures = self._to_device([s.temperature for s in seqs], torch.float32)
         logits = self.logits(seqs, is_prefill)
-        token_ids = self.sampler(logits, temperatures).tolist()
+        if all(s.temperature == 0 for s in seqs):
+            token_ids = logits.argmax(dim=-1).tolist()
+        else:
+            temperatures = self._to_device([s.temperature for s in seqs], torch.float32)
+            token_ids = self.sampler(logits, temperatures).tolist()
         return (token_ids, logits) if return_logits else token_ids

@@ -43,7 +43,7 @@ class TraceReplay:
         model = load_config(model_dir, dtype)
         ensure_libraries(model)
         requests, block = min(max(max_tokens, 1), cls.MAX_REQUESTS), EngineConfig.kvcache_block_size
-        return cls(EngineConfig(model=model, model_dir=model_dir, reuse_prefix=False, max_num_seqs=requests,
+        return cls(EngineConfig(model=model, model_dir=model_dir, reuse_prefix=False, max_num_seqs=requests, decode_graphs=False,
                                 num_kvcache_blocks=max(max_tokens, 1) // block + 1 + requests,
                                 max_num_batched_tokens=max(max_tokens, 1)))
 

@@ -178,3 +178,38 @@ def test_trace_runner_and_command_line(models, tmp_path):
     assert p.returncode == 0, p.stderr[-2000:]
     lines = [json.loads(l) for l in p.stdout.splitlines() if l.startswith("{")]
     assert len(lines) == 2 and lines[0]["token_ids"][0] == int(want[-1].argmax())
+
+
+@pytest.mark.parametrize("name,dtype", [("odd", "float32"), ("wide", "float32"), ("wide", "bfloat16"), ("plain", "bfloat16")])
+def test_recorded_decode_steps_equal_eager_ones(models, name, dtype):
+    """Every decode step of a batch whose size and contexts change, replayed from the recorded graphs, against the same
+    step run eagerly and (float32) against the oracle; eager prompts of new requests run between the replays."""
+    announce(f"feguvik {name} {dtype}: decode graphs")
+    path, cfg, w = models(name)
+    prompts = [draw_tokens(cfg, n, seed=40 + n) for n in (3, 60, 21, 9, 30)]
+    params = [SamplingParams(temperature=0.0, max_tokens=m, ignore_eos=True) for m in (60, 10, 25, 30, 8)]
+    logits = {}
+    for graphs in (True, False):
+        engine = LLMEngine(path, dtype=dtype, num_kvcache_blocks=40, max_num_seqs=3, max_num_batched_tokens=96, max_model_len=200,
+                           decode_graphs=graphs)
+        seen, first = {}, {}
+        def hook(seqs, is_prefill, rows):
+            for s, row in zip(seqs, rows.float().cpu()):
+                seen[(first.setdefault(s.seq_id, len(first)), len(s))] = (list(s.token_ids), row)
+        engine.step_hook = hook
+        engine.generate(prompts, params)
+        logits[graphs] = seen
+        if graphs:
+            g = engine.model_runner.graphs
+            assert g.replays >= 59 and g.recorded and all(r is not None for r in g.recorded.values()), g.recorded
+            assert len(g.recorded) >= 3                    # one, two and three sequences (padded to four)
+    close = 0
+    for key, (toks, row) in logits[True].items():
+        if dtype == "float32":
+            want = oracle_logits(toks, w, cfg)[-1]
+            assert float((row - want).abs().max() / want.std()) < F32_TOL * 5, key
+        other = logits[False].get(key)
+        if other is not None and other[0] == toks:
+            close += 1
+            assert float((row - other[1]).abs().max() / row.std()) < (1e-3 if dtype == "float32" else 0.5), key
+    assert close > len(logits[True]) // 2
