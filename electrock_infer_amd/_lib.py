@@ -45,7 +45,7 @@ EXPORTED_SYMBOLS = (
 
 # every function include/electrock_decoder.h declares
 DECODER_SYMBOLS = (
-    "ed_version", "ed_embed", "ed_residual_norm", "ed_relu_squared", "ed_token_gate",
+    "ed_version", "ed_embed", "ed_residual_norm", "ed_relu_squared", "ed_token_gate", "ed_skinny_gemm_splits", "ed_skinny_gemm",
     "ed_token_side_supported", "ed_token_side", "ed_gla_prefill", "ed_gla_step",
     "ed_latent_row_elems", "ed_latent_prepare", "ed_latent_paged", "ed_head_gemm", "ed_latent_gather",
     "ed_latent_prompt_supported", "ed_latent_prompt",
@@ -169,7 +169,9 @@ def load_decoder() -> ctypes.CDLL:
     signatures = {
         "ed_version": [],
         "ed_embed": [vp, vp, dbl, vp, vp, i64, i64, i32, i32, vp],
-        "ed_residual_norm": [i32, vp, vp, i32, vp, vp, vp, i64, i64, i32, dbl, i32, vp],
+        "ed_skinny_gemm_splits": [i64, i32, i32],
+        "ed_skinny_gemm": [vp, vp, vp, i32, i32, i64, i32, i32, i32, vp],
+        "ed_residual_norm": [i32, vp, vp, i32, i32, vp, vp, vp, i64, i64, i32, dbl, i32, vp],
         "ed_relu_squared": [vp, i64, i32, vp],
         "ed_token_gate": [vp, vp, vp, vp, i64, i32, vp, i64, i32, i32, i32, vp],
         "ed_token_side_supported": [i32, i32],

@@ -22,9 +22,14 @@ inline int allow_lds(const void* kernel, size_t bytes) {
 bool row_width_ok(int W);
 int launch_embed(const int32_t* tokens, const void* table, float scale, float* x, void* copy, int64_t copy_stride,
                  int64_t T, int W, int dtype, hipStream_t s);
-int launch_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
+int launch_residual_norm(int update, float* x, const void* y, int y_dtype, int y_parts, const float* post_w, const float* next_w,
                          void* out, int64_t out_stride, int64_t T, int W, float eps, int dtype, hipStream_t s);
 int launch_relu_squared(void* u, int64_t n, int dtype, hipStream_t s);
+
+// ---- skinny_gemm.hip ----
+bool skinny_supported(int64_t T, int N, int K);
+int skinny_splits(int T, int N, int K);
+int launch_skinny_gemm(const void* x, const void* w, void* out, bool f32, int splits, int T, int N, int K, int act, hipStream_t s);
 
 // ---- token_side.hip ----
 struct TokenSideProblem {

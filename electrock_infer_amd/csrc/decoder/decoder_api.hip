@@ -78,16 +78,17 @@ int ed_embed(const int32_t* tokens, const void* table, double scale, float* x, v
     return launch_embed(tokens, table, static_cast<float>(scale), x, copy, copy ? copy_stride : W, T, W, dtype, as_stream(stream));
 }
 
-int ed_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
+int ed_residual_norm(int update, float* x, const void* y, int y_dtype, int y_parts, const float* post_w, const float* next_w,
                      void* out, int64_t out_stride, int64_t T, int W, double eps, int dtype, void* stream) {
     if (!dtype_ok(dtype) || (update != 0 && y_dtype != dtype && y_dtype != EM_DTYPE_F32)) return EM_ERR_BAD_DTYPE;
+    if (y_parts < 1 || (y_parts > 1 && y_dtype != EM_DTYPE_F32)) return EM_ERR_BAD_SHAPE;
     if (update < 0 || update > 2 || T < 0 || T > kMaxRows || !row_width_ok(W) || (out && out_stride < W)) return EM_ERR_BAD_SHAPE;
     if (T == 0) return 0;
     if (!x || (update != 0 && !y) || (update == 1 && !post_w)) return EM_ERR_NULL_POINTER;
     // rows that are not a multiple of four elements go element by element
     if (W % 4 == 0 && (!aligned16(x) || !aligned16(y) || !aligned16(post_w) || !aligned16(next_w) || !aligned16(out)))
         return EM_ERR_ALIGNMENT;
-    return launch_residual_norm(update, x, y, update == 0 ? dtype : y_dtype, post_w, next_w, out, out ? out_stride : W, T, W,
+    return launch_residual_norm(update, x, y, update == 0 ? dtype : y_dtype, y_parts, post_w, next_w, out, out ? out_stride : W, T, W,
                                 static_cast<float>(eps), dtype, as_stream(stream));
 }
 
@@ -98,6 +99,21 @@ int ed_relu_squared(void* u, int64_t n, int dtype, void* stream) {
     if (!u) return EM_ERR_NULL_POINTER;
     if (!aligned16(u)) return EM_ERR_ALIGNMENT;
     return launch_relu_squared(u, n, dtype, as_stream(stream));
+}
+
+int ed_skinny_gemm_splits(int64_t T, int N, int K) { return skinny_supported(T, N, K) ? skinny_splits(static_cast<int>(T), N, K) : 0; }
+
+int ed_skinny_gemm(const void* x, const void* w, void* out, int out_dtype, int splits, int64_t T, int N, int K, int act,
+                   void* stream) {
+    if (!dtype_ok(out_dtype)) return EM_ERR_BAD_DTYPE;
+    if (T == 0) return 0;
+    if (!skinny_supported(T, N, K)) return EM_ERR_UNSUPPORTED;
+    if (splits < 1 || splits > 64 || splits > K / 64 || act < 0 || act > 1 ||
+        (splits > 1 && (act != 0 || out_dtype != EM_DTYPE_F32)))
+        return EM_ERR_BAD_SHAPE;
+    if (!x || !w || !out) return EM_ERR_NULL_POINTER;
+    if (!aligned16(x) || !aligned16(w)) return EM_ERR_ALIGNMENT;
+    return launch_skinny_gemm(x, w, out, out_dtype == EM_DTYPE_F32, splits, static_cast<int>(T), N, K, act, as_stream(stream));
 }
 
 int ed_token_gate(const void* x, const void* gate, const int32_t* tokens, const void* table, int64_t table_stride,

@@ -56,11 +56,12 @@ __global__ __launch_bounds__(256) void embed_kernel(const int32_t* __restrict__ 
 }
 
 // One workgroup per row.
+// y may be given as float32 partial sums [y_parts, T, W].
 //   UPDATE 0: x stays          UPDATE 1: x += y / rms(y) * post_w          UPDATE 2: x = y + post_w
 //   then, when out != null: out = next_w ? x / rms(x) * next_w : x, rounded to the compute type
 template <typename Elem, typename YElem, int UPDATE, int VEC, int THREADS>
 __global__ __launch_bounds__(THREADS) void residual_norm_kernel(
-    float* __restrict__ x, const typename YElem::storage* __restrict__ y, const float* __restrict__ post_w,
+    float* __restrict__ x, const typename YElem::storage* __restrict__ y, int y_parts, const float* __restrict__ post_w,
     const float* __restrict__ next_w, typename Elem::storage* __restrict__ out, int64_t out_stride, int W, float eps) {
     __shared__ float scratch[THREADS / kWave];
     constexpr int N = kRowMaxPerThread / VEC;
@@ -75,6 +76,12 @@ __global__ __launch_bounds__(THREADS) void residual_norm_kernel(
             const int c = (threadIdx.x + i * THREADS) * VEC;
             if (c < W) {
                 RowIo<YElem, VEC>::load(yr + c, v[i]);
+                for (int p = 1; p < y_parts; ++p) {
+                    float more[VEC];
+                    RowIo<YElem, VEC>::load(yr + static_cast<int64_t>(p) * gridDim.x * W + c, more);
+#pragma unroll
+                    for (int j = 0; j < VEC; ++j) v[i][j] += more[j];
+                }
 #pragma unroll
                 for (int j = 0; j < VEC; ++j) sum = fmaf(v[i][j], v[i][j], sum);
             }
@@ -156,26 +163,26 @@ __global__ __launch_bounds__(256) void relu_squared_kernel(typename Elem::storag
 }
 
 template <typename Elem, typename YElem, int UPDATE, int VEC>
-int launch_residual(float* x, const void* y, const float* post_w, const float* next_w, void* out, int64_t out_stride,
+int launch_residual(float* x, const void* y, int y_parts, const float* post_w, const float* next_w, void* out, int64_t out_stride,
                     int64_t T, int W, float eps, hipStream_t s) {
     typedef typename Elem::storage S;
     typedef typename YElem::storage YS;
     const dim3 grid(static_cast<unsigned>(T));
     if (W <= 256 * kRowMaxPerThread)
         launch((residual_norm_kernel<Elem, YElem, UPDATE, VEC, 256>), grid, dim3(256), 0, s, x,
-               static_cast<const YS*>(y), post_w, next_w, static_cast<S*>(out), out_stride, W, eps);
+               static_cast<const YS*>(y), y_parts, post_w, next_w, static_cast<S*>(out), out_stride, W, eps);
     else
         launch((residual_norm_kernel<Elem, YElem, UPDATE, VEC, 1024>), grid, dim3(1024), 0, s, x,
-               static_cast<const YS*>(y), post_w, next_w, static_cast<S*>(out), out_stride, W, eps);
+               static_cast<const YS*>(y), y_parts, post_w, next_w, static_cast<S*>(out), out_stride, W, eps);
     return launch_status();
 }
 
 template <typename Elem, typename YElem, int VEC>
-int dispatch_residual(int update, float* x, const void* y, const float* post_w, const float* next_w, void* out,
+int dispatch_residual(int update, float* x, const void* y, int y_parts, const float* post_w, const float* next_w, void* out,
                       int64_t out_stride, int64_t T, int W, float eps, hipStream_t s) {
-    if (update == 0) return launch_residual<Elem, YElem, 0, VEC>(x, y, post_w, next_w, out, out_stride, T, W, eps, s);
-    if (update == 1) return launch_residual<Elem, YElem, 1, VEC>(x, y, post_w, next_w, out, out_stride, T, W, eps, s);
-    return launch_residual<Elem, YElem, 2, VEC>(x, y, post_w, next_w, out, out_stride, T, W, eps, s);
+    if (update == 0) return launch_residual<Elem, YElem, 0, VEC>(x, y, y_parts, post_w, next_w, out, out_stride, T, W, eps, s);
+    if (update == 1) return launch_residual<Elem, YElem, 1, VEC>(x, y, y_parts, post_w, next_w, out, out_stride, T, W, eps, s);
+    return launch_residual<Elem, YElem, 2, VEC>(x, y, y_parts, post_w, next_w, out, out_stride, T, W, eps, s);
 }
 
 }  // namespace
@@ -200,12 +207,12 @@ int launch_embed(const int32_t* tokens, const void* table, float scale, float* x
     return launch_status();
 }
 
-int launch_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
+int launch_residual_norm(int update, float* x, const void* y, int y_dtype, int y_parts, const float* post_w, const float* next_w,
                          void* out, int64_t out_stride, int64_t T, int W, float eps, int dtype, hipStream_t s) {
     const bool vec = W % 4 == 0 && out_stride % 4 == 0;
 #define EM_RESIDUAL(E, Y)                                                                                        \
-    return vec ? dispatch_residual<E, Y, 4>(update, x, y, post_w, next_w, out, out_stride, T, W, eps, s)         \
-               : dispatch_residual<E, Y, 1>(update, x, y, post_w, next_w, out, out_stride, T, W, eps, s)
+    return vec ? dispatch_residual<E, Y, 4>(update, x, y, y_parts, post_w, next_w, out, out_stride, T, W, eps, s)         \
+               : dispatch_residual<E, Y, 1>(update, x, y, y_parts, post_w, next_w, out, out_stride, T, W, eps, s)
     if (dtype == EM_DTYPE_F32) { EM_RESIDUAL(F32Elem, F32Elem); }
     if (y_dtype == EM_DTYPE_F32) { EM_RESIDUAL(BF16Elem, F32Elem); }
     EM_RESIDUAL(BF16Elem, BF16Elem);

@@ -11,7 +11,7 @@ import torch
 import torch.nn.functional as F
 from torch import nn
 
-from ..layers.decoder_ops import ADD_NORMED, KEEP, REPLACE, embed_rows, linear_f32, residual_norm
+from ..layers.decoder_ops import ADD_NORMED, KEEP, REPLACE, embed_rows, linear_f32, linear_parts, residual_norm
 from ..layers.dense_mlp import DenseMLP
 from ..layers.gla import GatedLinearAttention
 from ..layers.latent_attention import LatentAttention
@@ -220,7 +220,7 @@ class FeguvikForCausalLM(nn.Module):
             if self.layer_hook is not None and r > 0:
                 self.layer_hook(r - 1, x)
             if opens_pass(r):
-                residual_norm(REPLACE, x, linear_f32(both, self.loop_in), self.loop_step[self.runs[r][1]], eps, h, norm)
+                residual_norm(REPLACE, x, linear_parts(both, self.loop_in, exact=True), self.loop_step[self.runs[r][1]], eps, h, norm)
 
         open_run(0, lambda out, norm: residual_norm(KEEP, x, None, None, eps, out, norm))
         for r, (i, _) in enumerate(self.runs):

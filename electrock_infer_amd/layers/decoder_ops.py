@@ -13,11 +13,46 @@ def _ptr(t: Optional[torch.Tensor]) -> Optional[int]:
     return None if t is None else t.data_ptr()
 
 
+def _skinny(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, splits: int, act: int) -> torch.Tensor:
+    (T, K), N = x.shape, weight.shape[0]
+    code = _lib.load_decoder().ed_skinny_gemm(x.data_ptr(), weight.data_ptr(), out.data_ptr(), _lib.dtype_code(out.dtype), splits,
+                                              T, N, K, act, _lib.current_stream(x.device))
+    _lib.check_decoder(code, "skinny_gemm")
+    return out
+
+
+def _skinny_splits(x: torch.Tensor, weight: torch.Tensor) -> int:
+    """For a decode batch that the weight-streaming kernel takes: how many ranges of K fill the chip; else 0."""
+    if x.dtype != torch.bfloat16 or x.shape[0] > 64 or not x.is_contiguous():
+        return 0
+    return _lib.load_decoder().ed_skinny_gemm_splits(x.shape[0], weight.shape[0], x.shape[1])
+
+
+def linear(x: torch.Tensor, weight: torch.Tensor, act: Optional[str] = None) -> torch.Tensor:
+    """act(x @ weight^T) in x's type: a weight-streaming kernel for a decode batch, a library product otherwise;
+    ``act``: None or 'relu_squared'."""
+    if _skinny_splits(x, weight):
+        return _skinny(x, weight, torch.empty(x.shape[0], weight.shape[0], dtype=x.dtype, device=x.device), 1, int(act is not None))
+    out = F.linear(x, weight)
+    return relu_squared_(out) if act is not None else out
+
+
 def linear_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
     """x @ weight^T with the float32 accumulators as the result, for sums that stay float32."""
     if x.dtype == torch.float32:
         return F.linear(x, weight)
+    if _skinny_splits(x, weight):
+        return _skinny(x, weight, torch.empty(x.shape[0], weight.shape[0], dtype=torch.float32, device=x.device), 1, 0)
     return torch.mm(x, weight.t(), out_dtype=torch.float32)
+
+
+def linear_parts(x: torch.Tensor, weight: torch.Tensor, exact: bool = False) -> torch.Tensor:
+    """x @ weight^T as ``residual_norm`` takes it: [T, N], or float32 partial sums [parts, T, N] of a decode batch.
+    ``exact``: not rounded to the compute type on the way."""
+    splits = _skinny_splits(x, weight)
+    if splits > 1:
+        return _skinny(x, weight, torch.empty(splits, x.shape[0], weight.shape[0], dtype=torch.float32, device=x.device), splits, 0)
+    return linear_f32(x, weight) if exact else linear(x, weight)
 
 
 def embed_rows(tokens: torch.Tensor, table: torch.Tensor, scale: float, copy: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -37,11 +72,13 @@ KEEP, ADD_NORMED, REPLACE = 0, 1, 2
 def residual_norm(update: int, x: torch.Tensor, y: Optional[torch.Tensor], post_w: Optional[torch.Tensor], eps: float,
                   out: Optional[torch.Tensor], next_w: Optional[torch.Tensor] = None) -> None:
     """Update the stream ``x`` in place (KEEP; ADD_NORMED: x += y / rms(y) * post_w; REPLACE: x = y + post_w) and write
-    the next sublayer's input into ``out`` (rows may be strided): x / rms(x) * next_w, or x itself, in out's type."""
+    the next sublayer's input into ``out`` (rows may be strided): x / rms(x) * next_w, or x itself, in out's type.
+    ``y`` [T, W] or partial sums [parts, T, W] (``linear_parts``)."""
     T, W = x.shape
+    parts = y.shape[0] if y is not None and y.dim() == 3 else 1
     dtype = out.dtype if out is not None else (y.dtype if y is not None else x.dtype)
     code = _lib.load_decoder().ed_residual_norm(
-        update, x.data_ptr(), _ptr(y), _lib.dtype_code(y.dtype if y is not None else dtype), _ptr(post_w), _ptr(next_w),
+        update, x.data_ptr(), _ptr(y), _lib.dtype_code(y.dtype if y is not None else dtype), parts, _ptr(post_w), _ptr(next_w),
         _ptr(out), out.stride(0) if out is not None else 0, T, W, float(eps), _lib.dtype_code(dtype),
         _lib.current_stream(x.device))
     _lib.check_decoder(code, "residual_norm")
@@ -97,7 +134,7 @@ class StackedLinear(torch.nn.Module):
         param.data[self.offset[name]:self.offset[name] + self.rows[name]].copy_(loaded)
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
-        return F.linear(x, self.weight)
+        return linear(x, self.weight)
 
     def section_ptr(self, out: torch.Tensor, name: str) -> int:
         return out.data_ptr() + self.offset[name] * out.element_size()

@@ -1,11 +1,10 @@
 """Gated linear attention (csrc/decoder/gla.hip): a recurrent mixer with one decay per key channel, a float32 state per
 head and sequence, a norm over every head's output and a SiLU gate."""
 import torch
-import torch.nn.functional as F
 from torch import nn
 
 from .. import _lib
-from .decoder_ops import StackedLinear, byref
+from .decoder_ops import StackedLinear, byref, linear_parts
 
 
 class GatedLinearAttention(nn.Module):
@@ -29,7 +28,7 @@ class GatedLinearAttention(nn.Module):
         return (self.heads, self.dim, self.vdim)
 
     def forward(self, h: torch.Tensor, batch, states: torch.Tensor) -> torch.Tensor:
-        """h [T, width] -> [T, width]; ``states`` float32 [slots, heads, dim, vdim] is updated in place."""
+        """h [T, width] -> [T, width] (as ``linear_parts`` has it); ``states`` float32 [slots, heads, dim, vdim] is updated in place."""
         T = h.shape[0]
         p = self.in_proj(h)
         out = torch.empty(T, self.heads * self.vdim, dtype=h.dtype, device=h.device)
@@ -52,4 +51,4 @@ class GatedLinearAttention(nn.Module):
                 cd = torch.empty(batch.n_chunks, self.heads * self.dim, dtype=torch.float32, device=h.device)
                 a.chunk_states, a.chunk_decay = cs.data_ptr(), cd.data_ptr()
             _lib.check_decoder(lib.ed_gla_prefill(byref(a), stream), "gla_prefill")
-        return F.linear(out, self.o)
+        return linear_parts(out, self.o)

@@ -5,7 +5,7 @@ import torch.nn.functional as F
 from torch import nn
 
 from .. import _lib
-from .decoder_ops import StackedLinear, byref, head_gemm, pad_k
+from .decoder_ops import StackedLinear, byref, head_gemm, linear_parts, pad_k
 
 
 def rotary_frequencies(dims: int, base: float) -> torch.Tensor:
@@ -51,7 +51,7 @@ class LatentAttention(nn.Module):
         return max(1, min(-(-self.TARGET_WORKGROUPS // groups), -(-batch.max_context // 128), 64))
 
     def forward(self, h: torch.Tensor, batch, cache: torch.Tensor) -> torch.Tensor:
-        """h [T, width] -> [T, width]; ``cache`` [blocks, block_size, row_elems] receives the new tokens' rows first."""
+        """h [T, width] -> [T, width] (as ``linear_parts`` has it); ``cache`` [blocks, block_size, row_elems] receives the new tokens' rows first."""
         T, dev = h.shape[0], h.device
         p = self.in_proj(h)
         a = _lib.LatentArgs(q=self.in_proj.section_ptr(p, "q"), q_stride=p.stride(0), down=self.in_proj.section_ptr(p, "dkv"),
@@ -68,7 +68,7 @@ class LatentAttention(nn.Module):
             self._attend_written_out(p, batch, cache, o)
         else:
             self._attend_paged(a, p, batch, o)
-        return F.linear(o, self.o)
+        return linear_parts(o, self.o)
 
     def writes_out(self, batch, dtype) -> bool:
         """A long portion: the up-projections of its context cost less than attending over the latents."""

@@ -25,15 +25,24 @@ int ed_version(void);
 int ed_embed(const int32_t* tokens, const void* table, double scale, float* x, void* copy, int64_t copy_stride,
              int64_t T, int W, int dtype, void* stream);
 
-/* Update of the float32 stream x [T, W] by a sublayer's result y [T, W] (y_dtype), then the next sublayer's input:
+/* Update of the float32 stream x [T, W] by a sublayer's result y [T, W] (y_dtype; or its float32 partial sums
+ * [y_parts, T, W]), then the next sublayer's input:
  *   update 0: x stays      1: x += y / sqrt(mean(y^2) + eps) * post_w      2: x = y + post_w (post_w may be null)
  *   out (may be null): next_w ? x / sqrt(mean(x^2) + eps) * next_w : x, rounded to dtype, rows out_stride apart.
  * post_w, next_w: float32 [W]. */
-int ed_residual_norm(int update, float* x, const void* y, int y_dtype, const float* post_w, const float* next_w,
-                     void* out, int64_t out_stride, int64_t T, int W, double eps, int dtype, void* stream);
+int ed_residual_norm(int update, float* x, const void* y, int y_dtype, int y_parts, const float* post_w,
+                     const float* next_w, void* out, int64_t out_stride, int64_t T, int W, double eps, int dtype, void* stream);
 
 /* u = max(u, 0)^2, n elements in place. */
 int ed_relu_squared(void* u, int64_t n, int dtype, void* stream);
+
+/* out = act(x w^T) for a decode batch, bf16 operands: x [T, K], w [N, K], T <= 64 (fewer for large
+ * weights), K a multiple of 64; act 0: none,
+ * 1: max(v, 0)^2.  splits > 1: out is float32 [splits, T, N], partial sums over K (no act).  ed_skinny_gemm_splits: how
+ * many fill the chip, 0 if the shape is not taken. */
+int ed_skinny_gemm_splits(int64_t T, int N, int K);
+int ed_skinny_gemm(const void* x, const void* w, void* out, int out_dtype, int splits, int64_t T, int N, int K, int act,
+                   void* stream);
 
 /* g [T, dim] = gelu_tanh(x gate^T) * table[tokens[t]][column0 + c]; x [T, W], gate [dim, W]. */
 int ed_token_gate(const void* x, const void* gate, const int32_t* tokens, const void* table, int64_t table_stride,

@@ -270,10 +270,16 @@ def test_decoder_argument_errors_are_reported_before_any_launch():
     assert lib.ed_embed(None, None, 1.0, None, None, 0, 4, 8, F16, None) == -3
     assert lib.ed_embed(None, None, 1.0, None, None, 0, 4, 1 << 20, BF16, None) == -2
     assert lib.ed_embed(None, None, 1.0, None, None, 0, 4, 8, BF16, None) == -1
-    assert lib.ed_residual_norm(3, None, None, BF16, None, None, None, 0, 1, 8, 1e-6, BF16, None) == -2
-    assert lib.ed_residual_norm(1, None, None, BF16, None, None, None, 0, 1, 8, 1e-6, F32, None) == -3
+    assert lib.ed_residual_norm(3, None, None, BF16, 1, None, None, None, 0, 1, 8, 1e-6, BF16, None) == -2
+    assert lib.ed_residual_norm(1, None, None, BF16, 1, None, None, None, 0, 1, 8, 1e-6, F32, None) == -3
     assert lib.ed_token_gate(None, None, None, None, 8, 4, None, 1, 16, 5, BF16, None) == -2           # columns 4 .. 8 of 8
+    assert lib.ed_residual_norm(1, None, None, BF16, 2, None, None, None, 0, 1, 8, 1e-6, BF16, None) == -2    # partial sums are float32
     assert lib.ed_relu_squared(None, 0, BF16, None) == 0
+    assert lib.ed_skinny_gemm_splits(65, 64, 64) == 0 and lib.ed_skinny_gemm_splits(33, 4096, 4096) == 0 and lib.ed_skinny_gemm_splits(4, 64, 100) == 0
+    assert lib.ed_skinny_gemm_splits(64, 2048, 2048) > 1 and lib.ed_skinny_gemm_splits(64, 64, 64) == 1
+    assert lib.ed_skinny_gemm(None, None, None, BF16, 2, 4, 64, 128, 0, None) == -2
+    assert lib.ed_skinny_gemm(None, None, None, BF16, 1, 4, 64, 128, 0, None) == -1
+    assert lib.ed_skinny_gemm(None, None, None, BF16, 1, 4, 64, 100, 0, None) == -4
     g = _lib.GlaArgs(n_seqs=1, heads=2, dim=300, vdim=8, rank=4, a2_stride=4, dtype=BF16, tau=1.0)
     assert lib.ed_gla_step(ctypes.byref(g), None) == -4
     g.dim = 8

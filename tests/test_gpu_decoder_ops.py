@@ -70,7 +70,8 @@ def test_feed_forward_and_token_side_input(dtype):
     w = {k: v.to(dtype).float() for k, v in w.items()}
     mlp, side = DenseMLP(W, ff, dtype).to(DEV), TokenSideInput(W, dim, layer * dim, dtype).to(DEV)
     mlp.up.data.copy_(w["up"]), mlp.down.data.copy_(w["down"])
-    close(mlp(to(x, dtype)), F.feed_forward(x.float(), w, "", {"kind": "dense"}), dtype)
+    y = mlp(to(x, dtype))
+    close(y.sum(0) if y.dim() == 3 else y, F.feed_forward(x.float(), w, "", {"kind": "dense"}), dtype)
     side.gate.data.copy_(w["l2.side.gate"]), side.proj.data.copy_(w["l2.side.proj"]), side.norm.data.copy_(w["l2.side.norm"])
     toks = torch.arange(T) * 5 % 30
     y = side(to(x, dtype), toks.int().to(DEV), to(w["side.embed"], dtype))
@@ -106,6 +107,24 @@ def test_end_of_a_layer_with_token_side_input(T, W, dim, dtype):
         rows = (xg.cpu() - ref).pow(2).mean(-1).sqrt()
         assert float(rows.max()) < (1e-4 if dtype == F32 else 5e-2)
     assert bool((both[:, W:] == 5).all())
+
+
+@pytest.mark.parametrize("T,N,K", [(1, 5, 64), (16, 300, 192), (17, 48, 640), (33, 33, 1024), (64, 2048, 2048), (32, 2048, 6144), (3, 9000, 128), (16, 9000, 128), (65, 40, 64), (7, 40, 72)])
+def test_decode_batch_products(T, N, K):
+    """The weight-streaming product in its three forms (and the library's, for shapes that it does not take)."""
+    announce(f"skinny gemm {T} {N} {K}")
+    x, w = rand(T, K, seed=1).to(BF16), rand(N, K, seed=2, scale=K ** -0.5).to(BF16)
+    ref = x.double() @ w.double().t()
+    xg, wg = to(x, BF16), to(w, BF16)
+    close(ops.linear(xg, wg), ref, BF16, bf16=4e-3)
+    close(ops.linear(xg, wg, "relu_squared"), F.relu_squared(ref), BF16, bf16=8e-3 if ops._skinny_splits(xg, wg) else 2e-2)
+    close(ops.linear_f32(xg, wg), ref, F32)
+    parts = ops.linear_parts(xg, wg, exact=True)
+    assert parts.dim() == (3 if ops._skinny_splits(xg, wg) > 1 else 2)
+    close(parts.sum(0) if parts.dim() == 3 else parts, ref, F32)
+    stream, out = torch.zeros(T, N, device=DEV), torch.empty(T, N, dtype=BF16, device=DEV)
+    ops.residual_norm(ops.ADD_NORMED, stream, parts, torch.ones(N, device=DEV), 1e-6, out)
+    close(stream, F.rms_norm(ref, torch.ones(N, dtype=torch.float64), 1e-6), F32)
 
 
 @pytest.mark.parametrize("dtype", [F32, BF16])
@@ -150,6 +169,7 @@ class Feed:
         batch = make_ragged([s for s, _, _ in live], BLOCK, self.chunk, DEV)
         h = torch.cat([h[s.num_computed_tokens:s.num_computed_tokens + n] for s, h, n in live])
         out = mixer(to(h, dtype), batch, cache).float().cpu()
+        out = out.sum(0) if out.dim() == 3 else out
         for s, _, n in live:
             s.num_computed_tokens += n
         return list(out.split([n for _, _, n in live]))
