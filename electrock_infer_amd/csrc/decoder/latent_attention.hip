@@ -59,7 +59,9 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentProblem p) {
 }
 
 // ---- per-head product  out[t, h, n] = sum_k a[t, h, k] b[h][n][k],  b's rows padded with zeros to 32 elements ----
-template <typename Elem, int MT>
+// A wave makes MT * 16 rows by 64 columns.  KSPLIT: the workgroup's four waves make the same tile, each from a quarter of
+// the k steps, and add up in LDS (few tiles of long rows); else they stand side by side along the columns.
+template <typename Elem, int MT, bool KSPLIT>
 __global__ __launch_bounds__(256) void head_gemm_kernel(const typename Elem::storage* __restrict__ a, int64_t a_row,
                                                         int64_t a_head, const typename Elem::storage* __restrict__ b,
                                                         typename Elem::storage* __restrict__ out, int64_t o_row,
@@ -69,9 +71,10 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const typename Elem::sto
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, lq = lane >> 4;
     const int h = blockIdx.z;
     const int64_t t0 = static_cast<int64_t>(blockIdx.x) * 16 * MT;
-    const int n0 = blockIdx.y * (blockDim.x / kWave) * 64 + wave * 64;
-    if (n0 >= N) return;
+    const int n0 = KSPLIT ? blockIdx.y * 64 : blockIdx.y * (blockDim.x / kWave) * 64 + wave * 64;
+    if (!KSPLIT && n0 >= N) return;
     const int KP = (K + 31) / 32 * 32;
+    const int k_begin = KSPLIT ? KP / 32 * wave / 4 * 32 : 0, k_end = KSPLIT ? KP / 32 * (wave + 1) / 4 * 32 : KP;
     const typename Elem::storage* bh = b + static_cast<int64_t>(h) * N * KP;
     f32x4_t acc[MT][NT];
 #pragma unroll
@@ -79,12 +82,12 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const typename Elem::sto
 #pragma unroll
         for (int n = 0; n < NT; ++n) acc[m][n] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
     constexpr int kSteps = MT == 4 ? 2 : 4;  // k steps whose operands are in flight together
-    for (int k0 = 0; k0 < KP; k0 += 32 * kSteps) {
+    for (int k0 = k_begin; k0 < k_end; k0 += 32 * kSteps) {
         typename M::frag fa[kSteps][MT], fb[kSteps][NT];
 #pragma unroll
         for (int u = 0; u < kSteps; ++u) {
             const int k = k0 + u * 32 + lq * 8;
-            if (k0 + u * 32 < KP) {
+            if (k0 + u * 32 < k_end) {
 #pragma unroll
                 for (int m = 0; m < MT; ++m) {
                     const int64_t t = t0 + m * 16 + l16;
@@ -99,12 +102,28 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const typename Elem::sto
         }
 #pragma unroll
         for (int u = 0; u < kSteps; ++u)
-            if (k0 + u * 32 < KP) {
+            if (k0 + u * 32 < k_end) {
 #pragma unroll
                 for (int m = 0; m < MT; ++m)
 #pragma unroll
                     for (int n = 0; n < NT; ++n) acc[m][n] = M::mac(fa[u][m], fb[u][n], acc[m][n]);
             }
+    }
+    if (KSPLIT) {
+        __shared__ float red[4][MT * 16 * 64];
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+#pragma unroll
+            for (int n = 0; n < NT; ++n)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) red[wave][(m * 16 + lq * 4 + r) * 64 + n * 16 + l16] = acc[m][n][r];
+        __syncthreads();
+        for (int i = threadIdx.x; i < MT * 16 * 64; i += 256) {
+            const int64_t t = t0 + i / 64;
+            const int col = n0 + i % 64;
+            if (t < T && col < N) out[t * o_row + h * o_head + col] = Elem::store(red[0][i] + red[1][i] + red[2][i] + red[3][i]);
+        }
+        return;
     }
 #pragma unroll
     for (int m = 0; m < MT; ++m)
@@ -433,17 +452,17 @@ int head_gemm(const void* a, int64_t a_row, int64_t a_head, const void* b, void*
     const int mt = ceil_div(T, 64) * cols * heads >= 512 ? 4 : T > 16 && ceil_div(T, 32) * cols * heads >= 256 ? 2 : 1;
     const int64_t wave_tiles = ceil_div(T, 16 * mt) * cols * heads;
     const int waves = static_cast<int>(wave_tiles >= 1024 ? (cols < 4 ? cols : 4) : 1);
+    const bool ksplit = waves == 1 && mt == 1 && K >= 256;
     const dim3 grid(static_cast<unsigned>(ceil_div(T, 16 * mt)), static_cast<unsigned>(ceil_div(N, waves * 64)),
-                    static_cast<unsigned>(heads)), block(static_cast<unsigned>(waves * kWave));
-    if (mt == 4)
-        launch((head_gemm_kernel<Elem, 4>), grid, block, 0, s, static_cast<const S*>(a), a_row, a_head,
-               static_cast<const S*>(b), static_cast<S*>(out), o_row, o_head, T, N, K, vec);
-    else if (mt == 2)
-        launch((head_gemm_kernel<Elem, 2>), grid, block, 0, s, static_cast<const S*>(a), a_row, a_head,
-               static_cast<const S*>(b), static_cast<S*>(out), o_row, o_head, T, N, K, vec);
-    else
-        launch((head_gemm_kernel<Elem, 1>), grid, block, 0, s, static_cast<const S*>(a), a_row, a_head,
-               static_cast<const S*>(b), static_cast<S*>(out), o_row, o_head, T, N, K, vec);
+                    static_cast<unsigned>(heads)), block(static_cast<unsigned>(ksplit ? 256 : waves * kWave));
+#define EM_HEAD_GEMM(MT, KS)                                                                                              \
+    launch((head_gemm_kernel<Elem, MT, KS>), grid, block, 0, s, static_cast<const S*>(a), a_row, a_head,                  \
+           static_cast<const S*>(b), static_cast<S*>(out), o_row, o_head, T, N, K, vec)
+    if (ksplit) EM_HEAD_GEMM(1, true);
+    else if (mt == 4) EM_HEAD_GEMM(4, false);
+    else if (mt == 2) EM_HEAD_GEMM(2, false);
+    else EM_HEAD_GEMM(1, false);
+#undef EM_HEAD_GEMM
     return launch_status();
 }
 

@@ -128,7 +128,7 @@ def test_decode_batch_products(T, N, K):
 
 
 @pytest.mark.parametrize("dtype", [F32, BF16])
-@pytest.mark.parametrize("T,H,N,K", [(1, 3, 5, 7), (16, 2, 64, 32), (17, 5, 70, 33), (90, 1, 300, 130)])
+@pytest.mark.parametrize("T,H,N,K", [(1, 3, 5, 7), (16, 2, 64, 32), (17, 5, 70, 33), (90, 1, 300, 130), (1, 2, 100, 512), (20, 3, 72, 300)])
 def test_head_gemm(T, H, N, K, dtype):
     announce(f"head gemm {T} {H} {N} {K} {dtype}")
     a, b = rand(T, H, K, seed=1).to(dtype), rand(H, N, K, seed=2).to(dtype)
