@@ -4,8 +4,9 @@ preemption, a prefix-reusing pool of cache blocks and a sampler -- this build's 
 Mixtral-shaped one and Feguvik.
 
 The Mixtral model exists to run the MoE path inside a whole generation loop (the end-to-end configuration of the
-benchmark) and its attention is not part of the hot path: it is torch's scaled_dot_product_attention over a gathered paged cache, the dense
-projections are torch matmuls; only the norms and the MoE block go through this package's own kernels.
+benchmark) and its attention is not part of the hot path: it is torch's scaled_dot_product_attention over a gathered
+paged cache, the dense projections are torch matmuls; only the norms and the MoE block go through this package's own
+kernels.
 """
 from .config import EngineConfig, ModelConfig, SamplingParams  # noqa: F401
 from .engine import LLMEngine  # noqa: F401

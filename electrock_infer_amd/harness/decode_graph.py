@@ -81,6 +81,9 @@ class DecodeGraphs:
         runner = self.runner
         return make_ragged(seqs, runner.block_size, runner.model.GLA_CHUNK, runner.device, padding=padding, into=into)
 
+    # (outside inference mode: a recording leaves tensors behind in torch's generator that later recordings write to)
+    @torch.inference_mode(False)
+    @torch.no_grad()
     def _record(self, batch_size: int, width: int) -> Optional[_Recorded]:
         runner, model = self.runner, self.runner.model
         padding = DecodePadding(batch_size, width, runner.config.num_kvcache_blocks, runner.config.num_state_slots)

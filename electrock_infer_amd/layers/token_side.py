@@ -9,7 +9,7 @@ from .decoder_ops import ADD_NORMED, linear, residual_norm, token_gate
 
 class TokenSideInput(nn.Module):
 
-    ONE_LAUNCH_ROWS = 6144
+    ONE_LAUNCH_ROWS = 2     # in widths: fewer rows do not fill the chip with the one-launch kernel's workgroups
 
     def __init__(self, width: int, dim: int, column0: int, dtype):
         super().__init__()
@@ -29,7 +29,7 @@ class TokenSideInput(nn.Module):
         prompt of a width its kernel takes; a few rows are better spread over the chip in four."""
         T, W = x.shape
         lib, dim = _lib.load_decoder(), self.gate.shape[0]
-        if T >= self.ONE_LAUNCH_ROWS and y.dim() == 2 and y.dtype == torch.bfloat16 and out.stride(0) % 4 == 0 and lib.ed_token_side_supported(W, dim) == 1:
+        if T >= self.ONE_LAUNCH_ROWS * W and y.dim() == 2 and y.dtype == torch.bfloat16 and out.stride(0) % 4 == 0 and lib.ed_token_side_supported(W, dim) == 1:
             code = lib.ed_token_side(x.data_ptr(), y.data_ptr(), post_w.data_ptr(), self.gate.data_ptr(), self.proj.data_ptr(),
                                      tokens.data_ptr(), table.data_ptr(), table.stride(0), self.column0, self.norm.data_ptr(),
                                      None if next_w is None else next_w.data_ptr(), out.data_ptr(), out.stride(0), T, W, dim,

@@ -96,7 +96,7 @@ def test_end_of_a_layer_with_token_side_input(T, W, dim, dtype):
     side = TokenSideInput(W, dim, layer * dim, dtype).to(DEV)
     side.gate.data.copy_(w["l1.side.gate"]), side.proj.data.copy_(w["l1.side.proj"]), side.norm.data.copy_(w["l1.side.norm"])
     both = torch.full((T, 2 * W), 5.0, dtype=dtype, device=DEV)
-    for next_w, out, one_launch in ((nxt, torch.empty(T, W, dtype=dtype, device=DEV), 1), (None, both[:, :W], 1),
+    for next_w, out, one_launch in ((nxt, torch.empty(T, W, dtype=dtype, device=DEV), 0), (None, both[:, :W], 0),
                                     (nxt, torch.empty(T, W, dtype=dtype, device=DEV), 10 ** 9)):
         xg, side.ONE_LAUNCH_ROWS = to(x), one_launch
         side.close_layer(xg, to(y, dtype), to(post), toks.int().to(DEV), to(w["side.embed"], dtype), eps, out,

@@ -112,3 +112,28 @@ def test_load_model_tp_shards(tmp_path):
             assert torch.equal(ex.w13_weight[e, :half], t[f"model.layers.0.block_sparse_moe.experts.{e}.w1.weight"][sl])
             assert torch.equal(ex.w13_weight[e, half:], t[f"model.layers.0.block_sparse_moe.experts.{e}.w3.weight"][sl])
             assert torch.equal(ex.w2_weight[e], t[f"model.layers.0.block_sparse_moe.experts.{e}.w2.weight"][:, sl])
+
+
+def test_whole_mixtral_checkpoint_loads(tmp_path):
+    """Every tensor name of a Mixtral checkpoint has its place in the engine's model; q, k and v are rows of one matrix."""
+    from electrock_infer_amd.harness import ModelConfig
+    from electrock_infer_amd.harness.model import MixtralForCausalLM
+    cfg = ModelConfig(vocab_size=40, hidden_size=32, intermediate_size=24, num_hidden_layers=2, num_attention_heads=4,
+                      num_key_value_heads=2, num_local_experts=4, max_position_embeddings=16)
+    t = _checkpoint(tmp_path, 4, 32, 24, extra=False)
+    g = torch.Generator().manual_seed(1)
+    draw = lambda *s: torch.randn(*s, generator=g).to(torch.bfloat16)
+    more = {"model.embed_tokens.weight": draw(40, 32), "model.norm.weight": draw(32), "lm_head.weight": draw(40, 32)}
+    for l in range(2):
+        pre = f"model.layers.{l}."
+        more.update({pre + "self_attn.q_proj.weight": draw(32, 32), pre + "self_attn.k_proj.weight": draw(16, 32),
+                     pre + "self_attn.v_proj.weight": draw(16, 32), pre + "self_attn.o_proj.weight": draw(32, 32),
+                     pre + "input_layernorm.weight": draw(32)})
+    save_file(more, str(tmp_path / "model-00003.safetensors"))
+    model = MixtralForCausalLM(cfg)
+    assert sorted(load_model(model, str(tmp_path))) == sorted({**t, **more})
+    for l, layer in enumerate(model.model.layers):
+        pre = f"model.layers.{l}.self_attn."
+        want = torch.cat([more[pre + f"{n}_proj.weight"] for n in "qkv"])
+        assert torch.equal(layer.self_attn.qkv_proj.weight, want)
+    assert torch.equal(model.lm_head.weight, more["lm_head.weight"])
