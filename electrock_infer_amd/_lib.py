@@ -45,8 +45,10 @@ EXPORTED_SYMBOLS = (
 
 # every function include/electrock_decoder.h declares
 DECODER_SYMBOLS = (
-    "ed_version", "ed_embed", "ed_residual_norm", "ed_relu_squared", "ed_token_gate", "ed_skinny_gemm_splits", "ed_skinny_gemm",
+    "ed_version", "ed_embed", "ed_residual_norm", "ed_relu_squared", "ed_silu_gate", "ed_gated_norm", "ed_token_gate", "ed_skinny_gemm_splits", "ed_skinny_gemm",
     "ed_token_side_supported", "ed_token_side", "ed_gla_prefill", "ed_gla_step",
+    "ed_recur_record", "ed_recur_prefill", "ed_recur_step",
+    "ed_attn_row_elems", "ed_attn_prepare", "ed_attn_paged", "ed_attn_prompt_supported", "ed_attn_prompt",
     "ed_latent_row_elems", "ed_latent_prepare", "ed_latent_paged", "ed_head_gemm", "ed_latent_gather",
     "ed_latent_prompt_supported", "ed_latent_prompt",
 )
@@ -60,6 +62,29 @@ class GlaArgs(ctypes.Structure):
                 [(n, ctypes.c_int32) for n in ("n_seqs", "n_chunks", "chunk_tokens", "heads", "dim", "vdim", "rank",
                                                "a2_stride", "dtype")] +
                 [(n, ctypes.c_float) for n in ("tau", "q_scale", "eps")])
+
+
+class RecurArgs(ctypes.Structure):
+    """Mirror of struct ed_recur_args."""
+    _fields_ = ([(n, ctypes.c_void_p) for n in ("q", "k", "v", "decay_in", "beta_in", "gate")] + [("stride", ctypes.c_int64)] +
+                [(n, ctypes.c_void_p) for n in ("conv_w", "conv_b", "a_log", "dt_bias", "skip", "norm_w", "ring", "states", "out",
+                                                "slots", "starts", "q_begin", "chunks", "seq_chunks", "q_rows", "k_rows",
+                                                "v_rows", "rates", "blocks", "chunk_states", "chunk_trans")] +
+                [(n, ctypes.c_int32) for n in ("n_seqs", "n_chunks", "chunk_tokens", "heads", "kv_heads", "dim", "vdim", "taps",
+                                               "dtype")] +
+                [(n, ctypes.c_float) for n in ("q_scale", "unit_eps", "eps")])
+
+
+class AttnArgs(ctypes.Structure):
+    """Mirror of struct ed_attn_args."""
+    _fields_ = ([(n, ctypes.c_void_p) for n in ("q", "k", "v")] + [("stride", ctypes.c_int64), ("v_first", ctypes.c_void_p),
+                                                                   ("v_first_stride", ctypes.c_int64)] +
+                [(n, ctypes.c_void_p) for n in ("mix", "q_norm", "k_norm", "inv_freq", "positions", "cache_rows", "cache", "q_rows",
+                                                "out", "q_begin", "starts", "tables", "part_o", "part_ml")] +
+                [("T", ctypes.c_int64)] +
+                [(n, ctypes.c_int32) for n in ("n_seqs", "max_q", "table_width", "block_size", "splits", "heads", "kv_heads", "dim",
+                                               "vdim", "rot", "window", "dtype")] +
+                [(n, ctypes.c_float) for n in ("scale", "softcap", "eps")])
 
 
 class LatentArgs(ctypes.Structure):
@@ -173,6 +198,16 @@ def load_decoder() -> ctypes.CDLL:
         "ed_skinny_gemm": [vp, vp, vp, i32, i32, i64, i32, i32, i32, vp],
         "ed_residual_norm": [i32, vp, vp, i32, i32, vp, vp, vp, i64, i64, i32, dbl, i32, vp],
         "ed_relu_squared": [vp, i64, i32, vp],
+        "ed_silu_gate": [vp, vp, i64, i32, i32, vp],
+        "ed_gated_norm": [vp, vp, i64, vp, i64, i32, i32, dbl, i32, vp],
+        "ed_recur_record": [i32],
+        "ed_recur_prefill": [ctypes.POINTER(RecurArgs), vp],
+        "ed_recur_step": [ctypes.POINTER(RecurArgs), vp],
+        "ed_attn_row_elems": [i32, i32, i32],
+        "ed_attn_prepare": [ctypes.POINTER(AttnArgs), vp],
+        "ed_attn_paged": [ctypes.POINTER(AttnArgs), vp],
+        "ed_attn_prompt_supported": [i32, i32],
+        "ed_attn_prompt": [ctypes.POINTER(AttnArgs), vp],
         "ed_token_gate": [vp, vp, vp, vp, i64, i32, vp, i64, i32, i32, i32, vp],
         "ed_token_side_supported": [i32, i32],
         "ed_token_side": [vp, vp, vp, vp, vp, vp, vp, i64, i32, vp, vp, vp, i64, i64, i32, i32, dbl, vp],

@@ -1,4 +1,5 @@
-// Shared declarations of the decoder library: float32-stream row kernels, gated linear attention, latent attention.
+// Shared declarations of the decoder library: float32-stream row kernels, gated linear attention, recurrences with one decay
+// per head, latent attention, softmax attention.
 #pragma once
 #include "../common.h"
 #include "../../../include/electrock_decoder.h"
@@ -25,6 +26,9 @@ int launch_embed(const int32_t* tokens, const void* table, float scale, float* x
 int launch_residual_norm(int update, float* x, const void* y, int y_dtype, int y_parts, const float* post_w, const float* next_w,
                          void* out, int64_t out_stride, int64_t T, int W, float eps, int dtype, hipStream_t s);
 int launch_relu_squared(void* u, int64_t n, int dtype, hipStream_t s);
+int launch_silu_gate(const void* u, void* out, int64_t T, int ff, int dtype, hipStream_t s);
+int launch_gated_norm(void* y, const void* z, int64_t z_stride, const float* w, int64_t T, int parts, int size, float eps, int dtype,
+                      hipStream_t s);
 
 // ---- skinny_gemm.hip ----
 bool skinny_supported(int64_t T, int N, int K);
@@ -75,6 +79,58 @@ bool gla_supported(int heads, int dim, int vdim, int rank);
 int launch_gla_prefill(const GlaProblem& g, const int32_t* seq_chunks, int n_chunks, int n_seqs, int chunk_tokens,
                        hipStream_t s);
 int launch_gla_step(const GlaProblem& g, int n_seqs, hipStream_t s);
+
+// ---- recurrence.hip ----
+struct RecurProblem {
+    const void *q, *k, *v;       // projections: q, k head g at g * dim, v head h at h * vdim
+    const void *decay_in, *beta_in, *gate;   // column h, column h (null: additive rule), head h at h * vdim (delta rule)
+    int64_t stride;              // of all of these
+    const float *conv_w, *conv_b;            // [channels, taps], [channels] or null; channels: q, k, v
+    const float *a_log, *dt_bias, *skip, *norm_w;   // [heads], [heads], [heads] or null, [vdim] (delta rule)
+    void* ring;                  // [slots, taps, channels]
+    float* states;               // [slots, heads, dim, vdim]
+    void* out;                   // [T, heads * vdim]
+    const int32_t *slots, *starts, *q_begin;
+    const int4* chunks;
+    const int32_t* seq_chunks;
+    float *q_f, *k_f;            // [T, kv_heads, dim padded to 16]
+    void* v_f;                   // [T, heads * vdim]
+    float *rates, *blocks, *chunk_states, *chunk_trans;
+    int n_seqs, n_chunks, chunk_tokens;
+    int heads, kv_heads, dim, vdim, taps, dtype;
+    float q_scale, unit_eps, eps;
+};
+bool recur_supported(int heads, int kv_heads, int dim, int vdim, int taps);
+__host__ __device__ constexpr int recur_record(bool delta) { return delta ? 576 : 320; }   // floats of a block's record
+int launch_recur_prefill(const RecurProblem& p, hipStream_t s);
+int launch_recur_step(const RecurProblem& p, hipStream_t s);
+
+// ---- attention.hip ----
+struct AttnProblem {
+    const void *q, *k, *v;       // projections, heads next to each other
+    int64_t stride;
+    const void* v_first;         // rows of the values that are mixed in
+    int64_t v_first_stride;
+    const float* mix;            // their share, a number in device memory; null: none
+    const float *q_norm, *k_norm;   // [dim] or null
+    const float* inv_freq;       // [rot / 2]
+    const int32_t *positions, *cache_rows;
+    void* cache;                 // [rows, attn_row_elems]
+    void* q_out;                 // [T, heads, attn_pitch(dim)]
+    void* out;                   // [T, heads * vdim]
+    const int32_t *q_begin, *starts, *tables;
+    int table_width, block_size;
+    int heads, kv_heads, dim, vdim, rot, window, dtype;
+    float scale, softcap, eps;
+};
+__host__ __device__ constexpr int attn_pitch(int dim) { return (dim + 7) / 8 * 8; }
+__host__ __device__ constexpr int attn_row_elems(int kv_heads, int dim, int vdim) { return kv_heads * (attn_pitch(dim) + attn_pitch(vdim)); }
+constexpr int kAttnMaxSplits = 64;
+bool attn_supported(int heads, int kv_heads, int dim, int vdim, int rot);
+bool attn_prompt_supported(int dim, int vdim);
+int launch_attn_prepare(const AttnProblem& p, int64_t T, hipStream_t s);
+int launch_attn_paged(const AttnProblem& p, int n_seqs, int max_q, int splits, float* part_o, float* part_ml, int64_t T, hipStream_t s);
+int launch_attn_prompt(const AttnProblem& p, int n_seqs, int max_q, hipStream_t s);
 
 // ---- latent_attention.hip ----
 struct LatentProblem {

@@ -61,11 +61,73 @@ int check_latent(const ed_latent_args* a) {
     return 0;
 }
 
+RecurProblem recur_problem(const ed_recur_args& a) {
+    RecurProblem p;
+    p.q = a.q; p.k = a.k; p.v = a.v;
+    p.decay_in = a.decay_in; p.beta_in = a.beta_in; p.gate = a.gate;
+    p.stride = a.stride;
+    p.conv_w = a.conv_w; p.conv_b = a.conv_b;
+    p.a_log = a.a_log; p.dt_bias = a.dt_bias; p.skip = a.skip; p.norm_w = a.norm_w;
+    p.ring = a.ring; p.states = a.states; p.out = a.out;
+    p.slots = a.slots; p.starts = a.starts; p.q_begin = a.q_begin;
+    p.chunks = reinterpret_cast<const int4*>(a.chunks); p.seq_chunks = a.seq_chunks;
+    p.q_f = a.q_rows; p.k_f = a.k_rows; p.v_f = a.v_rows;
+    p.rates = a.rates; p.blocks = a.blocks; p.chunk_states = a.chunk_states; p.chunk_trans = a.chunk_trans;
+    p.n_seqs = a.n_seqs; p.n_chunks = a.n_chunks; p.chunk_tokens = a.chunk_tokens;
+    p.heads = a.heads; p.kv_heads = a.kv_heads; p.dim = a.dim; p.vdim = a.vdim; p.taps = a.taps; p.dtype = a.dtype;
+    p.q_scale = a.q_scale; p.unit_eps = a.unit_eps; p.eps = a.eps;
+    return p;
+}
+
+int check_recur(const ed_recur_args* a) {
+    if (!a) return EM_ERR_NULL_POINTER;
+    if (!dtype_ok(a->dtype)) return EM_ERR_BAD_DTYPE;
+    if (a->n_seqs < 0 || a->n_seqs > kMaxSeqs) return EM_ERR_BAD_SHAPE;
+    if (!recur_supported(a->heads, a->kv_heads, a->dim, a->vdim, a->taps)) return EM_ERR_UNSUPPORTED;
+    if (a->n_seqs == 0) return 0;
+    if (!a->q || !a->k || !a->v || !a->decay_in || (a->beta_in && (!a->gate || !a->norm_w)) || !a->conv_w || !a->a_log || !a->dt_bias ||
+        !a->ring || !a->states || !a->out || !a->slots || !a->starts)
+        return EM_ERR_NULL_POINTER;
+    if (!aligned16(a->states) || !aligned16(a->ring)) return EM_ERR_ALIGNMENT;
+    return 0;
+}
+
+AttnProblem attn_problem(const ed_attn_args& a) {
+    AttnProblem p;
+    p.q = a.q; p.k = a.k; p.v = a.v;
+    p.stride = a.stride;
+    p.v_first = a.v_first; p.v_first_stride = a.v_first_stride; p.mix = a.mix;
+    p.q_norm = a.q_norm; p.k_norm = a.k_norm; p.inv_freq = a.inv_freq;
+    p.positions = a.positions; p.cache_rows = a.cache_rows;
+    p.cache = a.cache; p.q_out = a.q_rows; p.out = a.out;
+    p.q_begin = a.q_begin; p.starts = a.starts; p.tables = a.tables;
+    p.table_width = a.table_width; p.block_size = a.block_size;
+    p.heads = a.heads; p.kv_heads = a.kv_heads; p.dim = a.dim; p.vdim = a.vdim; p.rot = a.rot; p.window = a.window; p.dtype = a.dtype;
+    p.scale = a.scale; p.softcap = a.softcap; p.eps = a.eps;
+    return p;
+}
+
+int check_attn(const ed_attn_args* a, bool attend) {
+    if (!a) return EM_ERR_NULL_POINTER;
+    if (!dtype_ok(a->dtype)) return EM_ERR_BAD_DTYPE;
+    if (a->T < 0 || a->T > kMaxRows || a->window < 0 || !(a->softcap >= 0.0f)) return EM_ERR_BAD_SHAPE;
+    if (!attn_supported(a->heads, a->kv_heads, a->dim, a->vdim, a->rot)) return EM_ERR_UNSUPPORTED;
+    if (a->T == 0) return 0;
+    if (!a->cache || !a->q_rows) return EM_ERR_NULL_POINTER;
+    if (!aligned16(a->cache) || !aligned16(a->q_rows)) return EM_ERR_ALIGNMENT;
+    if (!attend) return 0;
+    if (a->n_seqs <= 0 || static_cast<int64_t>(a->n_seqs) * a->kv_heads > 65535 || a->max_q <= 0 || a->max_q > a->T || a->block_size <= 0 ||
+        a->table_width <= 0)
+        return EM_ERR_BAD_SHAPE;
+    if (!a->out || !a->q_begin || !a->starts || !a->tables) return EM_ERR_NULL_POINTER;
+    return 0;
+}
+
 }  // namespace
 
 extern "C" {
 
-int ed_version(void) { return 100; }
+int ed_version(void) { return 110; }
 
 int ed_embed(const int32_t* tokens, const void* table, double scale, float* x, void* copy, int64_t copy_stride,
              int64_t T, int W, int dtype, void* stream) {
@@ -101,6 +163,26 @@ int ed_relu_squared(void* u, int64_t n, int dtype, void* stream) {
     return launch_relu_squared(u, n, dtype, as_stream(stream));
 }
 
+int ed_silu_gate(const void* u, void* out, int64_t T, int ff, int dtype, void* stream) {
+    if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
+    if (T < 0 || T > kMaxRows || ff <= 0 || ff > (1 << 24)) return EM_ERR_BAD_SHAPE;
+    if (T == 0) return 0;
+    if (!u || !out) return EM_ERR_NULL_POINTER;
+    if (!aligned16(u) || !aligned16(out)) return EM_ERR_ALIGNMENT;
+    return launch_silu_gate(u, out, T, ff, dtype, as_stream(stream));
+}
+
+int ed_gated_norm(void* y, const void* z, int64_t z_stride, const float* w, int64_t T, int parts, int size, double eps, int dtype,
+                  void* stream) {
+    if (!dtype_ok(dtype)) return EM_ERR_BAD_DTYPE;
+    if (T < 0 || T > kMaxRows || parts <= 0 || parts > 65535 || !row_width_ok(size) || z_stride < static_cast<int64_t>(parts) * size)
+        return EM_ERR_BAD_SHAPE;
+    if (T == 0) return 0;
+    if (!y || !z || !w) return EM_ERR_NULL_POINTER;
+    if (!aligned16(y) || !aligned16(z) || !aligned16(w)) return EM_ERR_ALIGNMENT;
+    return launch_gated_norm(y, z, z_stride, w, T, parts, size, static_cast<float>(eps), dtype, as_stream(stream));
+}
+
 int ed_skinny_gemm_splits(int64_t T, int N, int K) { return skinny_supported(T, N, K) ? skinny_splits(static_cast<int>(T), N, K) : 0; }
 
 int ed_skinny_gemm(const void* x, const void* w, void* out, int out_dtype, int splits, int64_t T, int N, int K, int act,
@@ -108,8 +190,8 @@ int ed_skinny_gemm(const void* x, const void* w, void* out, int out_dtype, int s
     if (!dtype_ok(out_dtype)) return EM_ERR_BAD_DTYPE;
     if (T == 0) return 0;
     if (!skinny_supported(T, N, K)) return EM_ERR_UNSUPPORTED;
-    if (splits < 1 || splits > 64 || splits > K / 64 || act < 0 || act > 1 ||
-        (splits > 1 && (act != 0 || out_dtype != EM_DTYPE_F32)))
+    if (splits < 1 || splits > 64 || splits > K / 64 || act < 0 || act > 2 ||
+        (splits > 1 && (act != 0 || out_dtype != EM_DTYPE_F32)) || (act == 2 && out_dtype != EM_DTYPE_BF16))
         return EM_ERR_BAD_SHAPE;
     if (!x || !w || !out) return EM_ERR_NULL_POINTER;
     if (!aligned16(x) || !aligned16(w)) return EM_ERR_ALIGNMENT;
@@ -174,6 +256,57 @@ int ed_gla_step(const ed_gla_args* a, void* stream) {
     const int rc = check_gla(a);
     if (rc != 0 || a->n_seqs == 0) return rc;
     return launch_gla_step(gla_problem(*a), a->n_seqs, as_stream(stream));
+}
+
+int ed_recur_record(int delta) { return recur_record(delta != 0); }
+
+int ed_recur_prefill(const ed_recur_args* a, void* stream) {
+    const int rc = check_recur(a);
+    if (rc != 0 || a->n_seqs == 0) return rc;
+    if (a->n_chunks < a->n_seqs || a->chunk_tokens <= 0 || a->chunk_tokens % 16 != 0 || a->chunk_tokens / 16 > 65535) return EM_ERR_BAD_SHAPE;
+    if (!a->q_rows || !a->k_rows || !a->v_rows || !a->rates || !a->blocks || (a->n_chunks > a->n_seqs && (!a->chunk_states || !a->chunk_trans)))
+        return EM_ERR_WORKSPACE;
+    if (!a->q_begin || !a->chunks || !a->seq_chunks) return EM_ERR_NULL_POINTER;
+    if (!aligned16(a->chunks) || !aligned16(a->q_rows) || !aligned16(a->k_rows) || !aligned16(a->v_rows) || !aligned16(a->rates) ||
+        !aligned16(a->blocks) || !aligned16(a->chunk_states) || !aligned16(a->chunk_trans))
+        return EM_ERR_ALIGNMENT;
+    RecurProblem p = recur_problem(*a);
+    if (a->n_chunks == a->n_seqs) p.chunk_states = nullptr;
+    return launch_recur_prefill(p, as_stream(stream));
+}
+
+int ed_recur_step(const ed_recur_args* a, void* stream) {
+    const int rc = check_recur(a);
+    if (rc != 0 || a->n_seqs == 0) return rc;
+    return launch_recur_step(recur_problem(*a), as_stream(stream));
+}
+
+int ed_attn_row_elems(int kv_heads, int dim, int vdim) { return attn_row_elems(kv_heads, dim, vdim); }
+
+int ed_attn_prepare(const ed_attn_args* a, void* stream) {
+    const int rc = check_attn(a, false);
+    if (rc != 0 || a->T == 0) return rc;
+    if (!a->q || !a->k || !a->v || (a->mix && !a->v_first) || (a->rot > 0 && !a->inv_freq) || !a->positions || !a->cache_rows)
+        return EM_ERR_NULL_POINTER;
+    return launch_attn_prepare(attn_problem(*a), a->T, as_stream(stream));
+}
+
+int ed_attn_paged(const ed_attn_args* a, void* stream) {
+    const int rc = check_attn(a, true);
+    if (rc != 0 || a->T == 0) return rc;
+    if (a->splits < 1 || a->splits > kAttnMaxSplits) return EM_ERR_BAD_SHAPE;
+    if (a->splits > 1 && (!a->part_o || !a->part_ml)) return EM_ERR_WORKSPACE;
+    return launch_attn_paged(attn_problem(*a), a->n_seqs, a->max_q, a->splits, a->part_o, a->part_ml, a->T, as_stream(stream));
+}
+
+int ed_attn_prompt_supported(int dim, int vdim) { return attn_prompt_supported(dim, vdim) ? 1 : 0; }
+
+int ed_attn_prompt(const ed_attn_args* a, void* stream) {
+    const int rc = check_attn(a, true);
+    if (rc != 0 || a->T == 0) return rc;
+    if (!attn_prompt_supported(a->dim, a->vdim) || a->dtype != EM_DTYPE_BF16 || a->max_q > 128 * 65535) return EM_ERR_UNSUPPORTED;
+    if (!aligned16(a->out)) return EM_ERR_ALIGNMENT;
+    return launch_attn_prompt(attn_problem(*a), a->n_seqs, a->max_q, as_stream(stream));
 }
 
 int ed_latent_row_elems(int rank, int rot) { return latent_row_elems(rank, rot); }

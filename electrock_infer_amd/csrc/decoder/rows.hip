@@ -1,5 +1,5 @@
 // Row kernels of a decoder whose residual stream is float32: embedding, post-norm residual update fused with the next
-// layer's pre-norm, and squared ReLU.
+// layer's pre-norm, squared ReLU, gated SiLU, and the gated norm of a mixer's output.
 #include "decoder.h"
 
 namespace em {
@@ -162,6 +162,73 @@ __global__ __launch_bounds__(256) void relu_squared_kernel(typename Elem::storag
     RowIo<Elem, VEC>::store(u + i, v);
 }
 
+// out [T, ff] = silu(u[:, :ff]) * u[:, ff:]
+template <typename Elem, int VEC>
+__global__ __launch_bounds__(256) void silu_gate_kernel(const typename Elem::storage* __restrict__ u, typename Elem::storage* __restrict__ out,
+                                                        int64_t n, int ff) {
+    const int64_t i = (static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x) * VEC;
+    if (i >= n) return;
+    const int64_t row = i / ff, c = i - row * ff;
+    float g[VEC], v[VEC];
+    RowIo<Elem, VEC>::load(u + row * 2 * ff + c, g);
+    RowIo<Elem, VEC>::load(u + row * 2 * ff + ff + c, v);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] *= silu(g[j]);
+    RowIo<Elem, VEC>::store(out + i, v);
+}
+
+// y = y silu(z), normed in equal parts of `size` elements, times w, in place: one workgroup per (row, part)
+template <typename Elem, int VEC, int THREADS>
+__global__ __launch_bounds__(THREADS) void gated_norm_kernel(typename Elem::storage* __restrict__ y, const typename Elem::storage* __restrict__ z,
+                                                             int64_t z_stride, const float* __restrict__ w, int size, float eps) {
+    __shared__ float scratch[THREADS / kWave];
+    constexpr int N = kRowMaxPerThread / VEC;
+    const int64_t row = blockIdx.x;
+    const int c0 = blockIdx.y * size;
+    typename Elem::storage* yr = y + (row * gridDim.y + blockIdx.y) * size;
+    const typename Elem::storage* zr = z + row * z_stride + c0;
+    float v[N][VEC], sum = 0.0f;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        const int c = (threadIdx.x + i * THREADS) * VEC;
+        if (c < size) {
+            float g[VEC];
+            RowIo<Elem, VEC>::load(yr + c, v[i]);
+            RowIo<Elem, VEC>::load(zr + c, g);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) {
+                v[i][j] *= silu(g[j]);
+                sum = fmaf(v[i][j], v[i][j], sum);
+            }
+        }
+    }
+    const float rstd = 1.0f / sqrtf(block_sum<THREADS>(sum, scratch) / static_cast<float>(size) + eps);
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        const int c = (threadIdx.x + i * THREADS) * VEC;
+        if (c < size) {
+            float wv[VEC];
+            RowIo<F32Elem, VEC>::load(w + c0 + c, wv);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) v[i][j] *= rstd * wv[j];
+            RowIo<Elem, VEC>::store(yr + c, v[i]);
+        }
+    }
+}
+
+template <typename Elem, int VEC>
+int launch_gated(void* y, const void* z, int64_t z_stride, const float* w, int64_t T, int parts, int size, float eps, hipStream_t s) {
+    typedef typename Elem::storage S;
+    const dim3 grid(static_cast<unsigned>(T), static_cast<unsigned>(parts));
+    if (size <= 64 * kRowMaxPerThread / 4)
+        launch((gated_norm_kernel<Elem, VEC, 64>), grid, dim3(64), 0, s, static_cast<S*>(y), static_cast<const S*>(z), z_stride, w, size, eps);
+    else if (size <= 256 * kRowMaxPerThread)
+        launch((gated_norm_kernel<Elem, VEC, 256>), grid, dim3(256), 0, s, static_cast<S*>(y), static_cast<const S*>(z), z_stride, w, size, eps);
+    else
+        launch((gated_norm_kernel<Elem, VEC, 1024>), grid, dim3(1024), 0, s, static_cast<S*>(y), static_cast<const S*>(z), z_stride, w, size, eps);
+    return launch_status();
+}
+
 template <typename Elem, typename YElem, int UPDATE, int VEC>
 int launch_residual(float* x, const void* y, int y_parts, const float* post_w, const float* next_w, void* out, int64_t out_stride,
                     int64_t T, int W, float eps, hipStream_t s) {
@@ -230,6 +297,30 @@ int launch_relu_squared(void* u, int64_t n, int dtype, hipStream_t s) {
         else launch((relu_squared_kernel<F32Elem, 1>), grid, dim3(256), 0, s, static_cast<float*>(u), n);
     }
     return launch_status();
+}
+
+int launch_silu_gate(const void* u, void* out, int64_t T, int ff, int dtype, hipStream_t s) {
+    const int64_t n = T * ff;
+    const int vec = ff % 8 == 0 ? 8 : 1;
+    const dim3 grid(static_cast<unsigned>(ceil_div(ceil_div(n, vec), 256)));
+    if (dtype == EM_DTYPE_BF16) {
+        if (vec == 8) launch((silu_gate_kernel<BF16Elem, 8>), grid, dim3(256), 0, s, static_cast<const uint16_t*>(u), static_cast<uint16_t*>(out), n, ff);
+        else launch((silu_gate_kernel<BF16Elem, 1>), grid, dim3(256), 0, s, static_cast<const uint16_t*>(u), static_cast<uint16_t*>(out), n, ff);
+    } else {
+        if (vec == 8) launch((silu_gate_kernel<F32Elem, 8>), grid, dim3(256), 0, s, static_cast<const float*>(u), static_cast<float*>(out), n, ff);
+        else launch((silu_gate_kernel<F32Elem, 1>), grid, dim3(256), 0, s, static_cast<const float*>(u), static_cast<float*>(out), n, ff);
+    }
+    return launch_status();
+}
+
+int launch_gated_norm(void* y, const void* z, int64_t z_stride, const float* w, int64_t T, int parts, int size, float eps, int dtype,
+                      hipStream_t s) {
+    const bool vec = size % 4 == 0 && z_stride % 4 == 0;
+    if (dtype == EM_DTYPE_BF16)
+        return vec ? launch_gated<BF16Elem, 4>(y, z, z_stride, w, T, parts, size, eps, s)
+                   : launch_gated<BF16Elem, 1>(y, z, z_stride, w, T, parts, size, eps, s);
+    return vec ? launch_gated<F32Elem, 4>(y, z, z_stride, w, T, parts, size, eps, s)
+               : launch_gated<F32Elem, 1>(y, z, z_stride, w, T, parts, size, eps, s);
 }
 
 }  // namespace em

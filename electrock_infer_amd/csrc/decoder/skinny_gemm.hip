@@ -5,7 +5,8 @@
 // 64 elements of k a lane takes 32 consecutive bytes of one row (lane / 16 picks them, so that four lanes cover a
 // 128-byte line), for which the k order inside the step is permuted -- the token rows are read in the same order, and a
 // sum does not care.  The loads of four such steps are in flight at once.  With splits > 1 the results are float32
-// partial sums [splits, T, N] that the next kernel adds up.
+// partial sums [splits, T, N] that the next kernel adds up.  GLU: w is [2 N, K], a workgroup makes 16 columns of both
+// halves and stores silu(first) * second.
 #include "decoder.h"
 #include "mma.h"
 
@@ -16,15 +17,15 @@ constexpr int kWaves = 8;
 constexpr int kStepK = 64;
 constexpr int kAhead = 4;
 
-template <int MT, int NT, bool F32OUT>
+template <int MT, int NT, bool F32OUT, bool GLU = false>
 __global__ __launch_bounds__(kWaves * kWave, 2) void skinny_gemm_kernel(const uint16_t* __restrict__ x,
                                                                         const uint16_t* __restrict__ w, void* __restrict__ out,
                                                                         int T, int N, int K, int act) {
     typedef Mma<BF16Elem> M;
-    constexpr int kCols = 16 * NT, kTile = 16 * MT * kCols;
+    constexpr int kCols = 16 * NT, kTile = 16 * MT * kCols, kOutCols = GLU ? 16 : kCols;
     __shared__ float red[kWaves][kTile];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lq = lane >> 4;
-    const int n0 = blockIdx.x * kCols;
+    const int n0 = blockIdx.x * kOutCols;
     const int steps = K / kStepK, splits = gridDim.y, split = blockIdx.y;
     const int g0 = static_cast<int>(static_cast<int64_t>(steps) * split / splits);
     const int g1 = static_cast<int>(static_cast<int64_t>(steps) * (split + 1) / splits);
@@ -33,8 +34,8 @@ __global__ __launch_bounds__(kWaves * kWave, 2) void skinny_gemm_kernel(const ui
     const uint16_t* wr[NT];
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
-        const int c = n0 + n * 16 + l16;
-        wr[n] = w + static_cast<int64_t>(c < N ? c : N - 1) * K + lq * 16;   // (columns beyond N are not stored)
+        const int c = n0 + (GLU ? 0 : n * 16) + l16;
+        wr[n] = w + (static_cast<int64_t>(c < N ? c : N - 1) + (GLU ? n * static_cast<int64_t>(N) : 0)) * K + lq * 16;   // (columns beyond N are not stored)
     }
     const uint16_t* xr[MT];
 #pragma unroll
@@ -86,6 +87,20 @@ __global__ __launch_bounds__(kWaves * kWave, 2) void skinny_gemm_kernel(const ui
 #pragma unroll
             for (int r = 0; r < 4; ++r) red[wave][(m * 16 + lq * 4 + r) * kCols + n * 16 + l16] = acc[m][n][r];
     __syncthreads();
+    if (GLU) {
+        for (int i = tid; i < 16 * MT * 16; i += kWaves * kWave) {
+            const int t = i / 16, c = i % 16;
+            if (t >= T || n0 + c >= N) continue;
+            float g = 0.0f, u = 0.0f;
+#pragma unroll
+            for (int k = 0; k < kWaves; ++k) {
+                g += red[k][t * kCols + c];
+                u += red[k][t * kCols + 16 + c];
+            }
+            static_cast<uint16_t*>(out)[static_cast<int64_t>(t) * N + n0 + c] = f32_to_bf16_bits(silu(g) * u);
+        }
+        return;
+    }
     for (int i = tid; i < kTile; i += kWaves * kWave) {
         const int t = i / kCols, c = n0 + i % kCols;
         if (t >= T || c >= N) continue;
@@ -100,6 +115,12 @@ __global__ __launch_bounds__(kWaves * kWave, 2) void skinny_gemm_kernel(const ui
         if (F32OUT) static_cast<float*>(out)[at] = v;
         else static_cast<uint16_t*>(out)[at] = f32_to_bf16_bits(v);
     }
+}
+
+template <int MT>
+int launch_glu(const uint16_t* x, const uint16_t* w, void* out, int T, int N, int K, hipStream_t s) {
+    launch((skinny_gemm_kernel<MT, 2, false, true>), dim3(static_cast<unsigned>(ceil_div(N, 16))), dim3(kWaves * kWave), 0, s, x, w, out, T, N, K, 0);
+    return launch_status();
 }
 
 template <int MT, int NT>
@@ -135,6 +156,7 @@ int skinny_splits(int T, int N, int K) {
 int launch_skinny_gemm(const void* x, const void* w, void* out, bool f32, int splits, int T, int N, int K, int act, hipStream_t s) {
     const uint16_t* xp = static_cast<const uint16_t*>(x);
     const uint16_t* wp = static_cast<const uint16_t*>(w);
+    if (act == 2) return T <= 16 ? launch_glu<1>(xp, wp, out, T, N, K, s) : T <= 32 ? launch_glu<2>(xp, wp, out, T, N, K, s) : launch_glu<4>(xp, wp, out, T, N, K, s);
     if (cols_per_group(T, N) == 16) return launch_skinny<1, 1>(xp, wp, out, f32, splits, T, N, K, act, s);
     if (T <= 16) return launch_skinny<1, 2>(xp, wp, out, f32, splits, T, N, K, act, s);
     if (T <= 32) return launch_skinny<2, 2>(xp, wp, out, f32, splits, T, N, K, act, s);

@@ -1,7 +1,7 @@
 """The engine: decoder-only models, a paged cache and recurrent-state slots, a prefill-first batch planner with
 preemption, a prefix-reusing pool of cache blocks and a sampler -- this build's own counterpart of the reference's engine
 (electrock_infer/engine/*, models/mixtral.py, layers/sampler.py), kept small.  registry.py lists the models: a
-Mixtral-shaped one and Feguvik.
+Mixtral-shaped one, Feguvik and Nunivik.
 
 The Mixtral model exists to run the MoE path inside a whole generation loop (the end-to-end configuration of the
 benchmark) and its attention is not part of the hot path: it is torch's scaled_dot_product_attention over a gathered
@@ -11,5 +11,6 @@ kernels.
 from .config import EngineConfig, ModelConfig, SamplingParams  # noqa: F401
 from .engine import LLMEngine  # noqa: F401
 from .feguvik import FeguvikConfig, FeguvikForCausalLM  # noqa: F401
+from .nunivik import NunivikConfig, NunivikForCausalLM  # noqa: F401
 
 LLM = LLMEngine

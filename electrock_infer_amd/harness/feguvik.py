@@ -11,12 +11,13 @@ import torch
 import torch.nn.functional as F
 from torch import nn
 
-from ..layers.decoder_ops import ADD_NORMED, KEEP, REPLACE, embed_rows, linear_f32, linear_parts, residual_norm
+from ..layers.decoder_ops import ADD_NORMED, KEEP, REPLACE, embed_rows, linear_parts, residual_norm
 from ..layers.dense_mlp import DenseMLP
 from ..layers.gla import GatedLinearAttention
 from ..layers.latent_attention import LatentAttention
 from ..layers.token_side import TokenSideInput
 from .batch import RaggedBatch
+from .decoder_model import DecoderModel
 
 
 @dataclass
@@ -100,6 +101,11 @@ class FeguvikLayer(nn.Module):
         self.side = TokenSideInput(cfg.width, cfg.side_dim, index * cfg.side_dim, dtype) if cfg.side_dim else None
         self.post1 = self.post2 = None
 
+    def tensor_names(self) -> List[str]:
+        names = ["norm1", "norm1b", "ls1"] + [f"mix.{n}" for n in self.mix.TENSORS]
+        names += ["norm2", "norm2b", "ls2"] + [f"mlp.{n}" for n in self.mlp.TENSORS] if self.mlp is not None else []
+        return names + (["side.gate", "side.proj", "side.norm"] if self.side is not None else [])
+
     def finish_loading(self) -> None:
         """The output norm's weight and the layer scale multiply the same vector: one factor."""
         self.post1 = (self.norm1b * self.ls1).contiguous()
@@ -109,10 +115,11 @@ class FeguvikLayer(nn.Module):
             self.mix.finish_loading()
 
 
-class FeguvikForCausalLM(nn.Module):
+class FeguvikForCausalLM(DecoderModel):
 
-    ragged_batches = True
-    GLA_CHUNK = 256         # tokens that one workgroup of the linear attention's prompt kernel takes
+    NAMES = {"embed": "embed", "side.embed": "side_embed", "loop.in": "loop_in", "loop.step": "loop_step",
+             "final.norm": "final_norm", "head": "head"}
+    ZEROS = ("sink", "a2_bias")
 
     def __init__(self, cfg: FeguvikConfig):
         super().__init__()
@@ -129,74 +136,6 @@ class FeguvikForCausalLM(nn.Module):
         self.final_norm = nn.Parameter(torch.ones(W, dtype=torch.float32), requires_grad=False)
         self.head = matrix(cfg.vocab_size, W)
         self.runs = cfg.runs()
-        self.caches: List[torch.Tensor] = []      # per run: pages of the latent attention or states of the linear one
-        self.layer_hook = None                    # called as hook(run index, stream) behind every layer run when set
-
-    # ---- weights ----
-    _NAMES = {"embed": "embed", "side.embed": "side_embed", "loop.in": "loop_in", "loop.step": "loop_step",
-              "final.norm": "final_norm", "head": "head"}
-
-    def checkpoint_target(self, name: str):
-        """(parameter name, section or None) of a checkpoint tensor, or None."""
-        if name in self._NAMES:
-            return self._NAMES[name], None
-        first, _, rest = name.partition(".")
-        if first[:1] == "l" and first[1:].isdigit() and int(first[1:]) < len(self.layers):
-            prefix = f"layers.{first[1:]}."
-            if not rest.startswith("mix."):
-                return prefix + rest, None
-            entry = self.layers[int(first[1:])].mix.TENSORS.get(rest[4:])
-            if entry is not None:
-                return prefix + "mix." + entry[0], entry[1]
-        return None
-
-    def expected_tensors(self) -> List[str]:
-        """Checkpoint names of every parameter (section)."""
-        cfg, out = self.cfg, ["embed", "final.norm", "head"]
-        out += ["side.embed"] if cfg.side_dim else []
-        out += ["loop.in", "loop.step"] if cfg.loop is not None else []
-        for i, layer in enumerate(self.layers):
-            names = ["norm1", "norm1b", "ls1"] + [f"mix.{n}" for n in layer.mix.TENSORS]
-            names += ["norm2", "norm2b", "ls2", "mlp.up", "mlp.down"] if layer.mlp is not None else []
-            names += ["side.gate", "side.proj", "side.norm"] if layer.side is not None else []
-            out += [f"l{i}.{n}" for n in names]
-        return out
-
-    def finish_loading(self) -> None:
-        for layer in self.layers:
-            layer.finish_loading()
-
-    @torch.no_grad()
-    def init_random_weights(self, seed: int = 0, std: float = 0.02) -> None:
-        """N(0, std) for every matrix, ones for norms and layer scales, zeros for sinks and the decay's bias."""
-        g = torch.Generator(device=self.head.device).manual_seed(seed)
-        for name, p in self.named_parameters():
-            if p.dim() >= 2:
-                p.copy_(torch.randn(p.shape, generator=g, device=p.device, dtype=torch.float32) * std)
-            else:
-                p.fill_(0.0 if name.endswith(("sink", "a2_bias")) else 1.0)
-        self.finish_loading()
-
-    # ---- cache and state ----
-    def cache_bytes(self, block_size: int) -> Tuple[int, int]:
-        """(bytes of a cache block, bytes of a state slot), over all layer runs."""
-        block = slot = 0
-        for i, _ in self.runs:
-            mix = self.layers[i].mix
-            if isinstance(mix, LatentAttention):
-                block += block_size * mix.row_elems() * self.head.element_size()
-            else:
-                slot += mix.heads * mix.dim * mix.vdim * 4
-        return block, slot
-
-    def allocate_cache(self, num_blocks: int, block_size: int, num_slots: int, device) -> None:
-        self.caches = []
-        for i, _ in self.runs:
-            mix = self.layers[i].mix
-            if isinstance(mix, LatentAttention):
-                self.caches.append(torch.zeros(num_blocks, block_size, mix.row_elems(), dtype=self.head.dtype, device=device))
-            else:
-                self.caches.append(torch.zeros(num_slots, *mix.state_shape(), dtype=torch.float32, device=device))
 
     # ---- forward ----
     def forward(self, batch: RaggedBatch) -> torch.Tensor:
@@ -234,7 +173,3 @@ class FeguvikForCausalLM(nn.Module):
             else:
                 open_run(r + 1, lambda out, norm: residual_norm(ADD_NORMED, x, y, post, eps, out, norm))
         return h
-
-    def compute_logits(self, hidden: torch.Tensor, batch: RaggedBatch) -> torch.Tensor:
-        """float32 logits of the batch's wanted rows."""
-        return linear_f32(hidden.index_select(0, batch.logit_rows), self.head)

@@ -68,9 +68,11 @@ def _register_all() -> None:
     from .config import ModelConfig
     from .feguvik import FeguvikConfig, FeguvikForCausalLM
     from .model import MixtralForCausalLM
+    from .nunivik import NunivikConfig, NunivikForCausalLM
     register("MixtralForCausalLM", ModelConfig, lambda c: MixtralForCausalLM(c.model, fused_moe_tail=c.fused_moe_tail),
              _build.ensure_moe)
     register("Feguvik", FeguvikConfig, lambda c: FeguvikForCausalLM(c.model), _build.ensure_decoder)
+    register("Nunivik", NunivikConfig, lambda c: NunivikForCausalLM(c.model), _build.ensure_decoder)
 
 
 _register_all()

@@ -37,6 +37,21 @@ def linear(x: torch.Tensor, weight: torch.Tensor, act: Optional[str] = None) -> 
     return relu_squared_(out) if act is not None else out
 
 
+def linear_silu_gate(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """silu(x @ gate^T) * (x @ up^T) for ``weight`` = [gate; up]: one launch for a decode batch."""
+    (T, _), ff = x.shape, weight.shape[0] // 2
+    out = torch.empty(T, ff, dtype=x.dtype, device=x.device)
+    if _skinny_splits(x, weight):
+        code = _lib.load_decoder().ed_skinny_gemm(x.data_ptr(), weight.data_ptr(), out.data_ptr(), _lib.dtype_code(out.dtype), 1, T, ff,
+                                                  x.shape[1], 2, _lib.current_stream(x.device))
+        _lib.check_decoder(code, "skinny_gemm")
+        return out
+    u = F.linear(x, weight)
+    _lib.check_decoder(_lib.load_decoder().ed_silu_gate(u.data_ptr(), out.data_ptr(), T, ff, _lib.dtype_code(x.dtype),
+                                                        _lib.current_stream(x.device)), "silu_gate")
+    return out
+
+
 def linear_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
     """x @ weight^T with the float32 accumulators as the result, for sums that stay float32."""
     if x.dtype == torch.float32:
@@ -90,6 +105,15 @@ def relu_squared_(u: torch.Tensor) -> torch.Tensor:
     return u
 
 
+def gated_norm_(y: torch.Tensor, z_ptr: int, z_stride: int, weight: torch.Tensor, parts: int, eps: float) -> torch.Tensor:
+    """y = y * silu(z), RMS-normed in equal parts of a row, times ``weight``; in place."""
+    T, inner = y.shape
+    code = _lib.load_decoder().ed_gated_norm(y.data_ptr(), z_ptr, z_stride, weight.data_ptr(), T, parts, inner // parts, float(eps),
+                                             _lib.dtype_code(y.dtype), _lib.current_stream(y.device))
+    _lib.check_decoder(code, "gated_norm")
+    return y
+
+
 def token_gate(x: torch.Tensor, gate: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, column0: int) -> torch.Tensor:
     """gelu_tanh(x @ gate^T) * table[tokens, column0 : column0 + dim]"""
     (T, W), dim = x.shape, gate.shape[0]
@@ -114,24 +138,42 @@ def head_gemm(a: torch.Tensor, a_row: int, a_head: int, b: torch.Tensor, K: int,
     _lib.check_decoder(code, "head_gemm")
 
 
-class StackedLinear(torch.nn.Module):
-    """Several projections of one input as a single matrix: ``sections`` name -> rows, every section starting at a
-    multiple of eight rows (zeros between), so that vector loads of a section's outputs are aligned."""
+class StackedRows:
+    """Places of several named sections in one parameter: ``sections`` name -> rows, every section starting at a multiple of
+    ``align`` rows.  A checkpoint tensor that holds several sections one behind the other is loaded as 'first|second|...'."""
 
-    def __init__(self, width: int, sections, dtype):
-        super().__init__()
+    def __init__(self, sections, align: int = 1):
         self.offset, self.rows, at = {}, dict(sections), 0
         for name, rows in self.rows.items():
             self.offset[name] = at
-            at += (rows + 7) // 8 * 8
-        self.out_rows = at
-        self.weight = torch.nn.Parameter(torch.zeros(at, width, dtype=dtype), requires_grad=False)
-        self.weight.weight_loader = self.load_section
+            at += -(-rows // align) * align
+        self.total = at
 
-    def load_section(self, param, loaded: torch.Tensor, name: str) -> None:
-        if loaded.shape != (self.rows[name], param.shape[1]):
-            raise ValueError(f"projection '{name}' is {tuple(loaded.shape)}, expected {(self.rows[name], param.shape[1])}")
-        param.data[self.offset[name]:self.offset[name] + self.rows[name]].copy_(loaded)
+    def parameter(self, *columns, dtype) -> torch.nn.Parameter:
+        p = torch.nn.Parameter(torch.zeros(self.total, *columns, dtype=dtype), requires_grad=False)
+        p.weight_loader = self.load
+        return p
+
+    def load(self, param, loaded: torch.Tensor, names: str) -> None:
+        names = names.split("|")
+        if loaded.shape != (sum(self.rows[n] for n in names), *param.shape[1:]):
+            raise ValueError(f"projection '{'|'.join(names)}' is {tuple(loaded.shape)}, expected "
+                             f"{(sum(self.rows[n] for n in names), *param.shape[1:])}")
+        at = 0
+        for n in names:
+            param.data[self.offset[n]:self.offset[n] + self.rows[n]].copy_(loaded[at:at + self.rows[n]])
+            at += self.rows[n]
+
+
+class StackedLinear(torch.nn.Module):
+    """Several projections of one input as a single matrix.  A section starts at a multiple of eight rows (zeros between),
+    so that vector loads of its outputs are aligned."""
+
+    def __init__(self, width: int, sections, dtype):
+        super().__init__()
+        self.places = StackedRows(sections, 8)
+        self.offset, self.rows, self.out_rows = self.places.offset, self.places.rows, self.places.total
+        self.weight = self.places.parameter(width, dtype=dtype)
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         return linear(x, self.weight)

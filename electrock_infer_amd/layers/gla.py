@@ -24,6 +24,13 @@ class GatedLinearAttention(nn.Module):
     TENSORS = {**{n: ("in_proj.weight", n) for n in ("q", "k", "v", "g", "a1")}, "a2": ("a2", None),
                "a2.b": ("a2_bias", None), "norm": ("norm", None), "o": ("o", None)}
 
+    def cache_bytes(self, block_size: int):
+        """(bytes of a cache block, bytes of a state slot)"""
+        return 0, self.heads * self.dim * self.vdim * 4
+
+    def new_cache(self, num_blocks: int, block_size: int, num_slots: int, device) -> torch.Tensor:
+        return torch.zeros(num_slots, *self.state_shape(), dtype=torch.float32, device=device)
+
     def state_shape(self):
         return (self.heads, self.dim, self.vdim)
 

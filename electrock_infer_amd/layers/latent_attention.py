@@ -8,9 +8,9 @@ from .. import _lib
 from .decoder_ops import StackedLinear, byref, head_gemm, linear_parts, pad_k
 
 
-def rotary_frequencies(dims: int, base: float) -> torch.Tensor:
-    """base^(-2i / dims) for i < dims / 2, rounded once to float32."""
-    return (float(base) ** (-torch.arange(0, dims, 2, dtype=torch.float64) / max(dims, 1))).float()
+def rotary_frequencies(dims: int, base: float, factor: float = 1.0) -> torch.Tensor:
+    """base^(-2i / dims) / factor for i < dims / 2, rounded once to float32."""
+    return (float(base) ** (-torch.arange(0, dims, 2, dtype=torch.float64) / max(dims, 1)) / factor).float()
 
 
 class LatentAttention(nn.Module):
@@ -41,6 +41,13 @@ class LatentAttention(nn.Module):
         self.inv_freq.copy_(rotary_frequencies(self.rot, self.rotary_base))
         self.uk_t = pad_k(self.uk.data.view(self.heads, self.dim, self.rank).transpose(1, 2))
         self.uv_p = pad_k(self.uv.data.view(self.heads, self.vdim, self.rank))
+
+    def cache_bytes(self, block_size: int):
+        """(bytes of a cache block, bytes of a state slot)"""
+        return block_size * self.row_elems() * self.uk.element_size(), 0
+
+    def new_cache(self, num_blocks: int, block_size: int, num_slots: int, device) -> torch.Tensor:
+        return torch.zeros(num_blocks, block_size, self.row_elems(), dtype=self.uk.dtype, device=device)
 
     def row_elems(self) -> int:
         """Elements that one token takes in the cache."""

@@ -1,6 +1,7 @@
 /*
  * electrock_decoder.h — C ABI of libelectrock_decoder.so (MI355X / gfx950): the kernels of decoders whose residual
- * stream is float32 (row kernels), of gated linear attention and of latent attention over a paged cache.
+ * stream is float32 (row kernels), of gated linear attention, of recurrences with one decay per head, and of latent and
+ * softmax attention over a paged cache.
  *
  * Same conventions as electrock_moe.h: raw DEVICE pointers, plain sizes, a HIP stream passed as void*; asynchronous,
  * no allocation, no retained state; the device that owns the pointers is current.  Returns 0, an EM_ERR_* code (nothing
@@ -36,9 +37,17 @@ int ed_residual_norm(int update, float* x, const void* y, int y_dtype, int y_par
 /* u = max(u, 0)^2, n elements in place. */
 int ed_relu_squared(void* u, int64_t n, int dtype, void* stream);
 
+/* out [T, ff] = silu(u[t][c]) * u[t][ff + c]; u [T, 2 ff]. */
+int ed_silu_gate(const void* u, void* out, int64_t T, int ff, int dtype, void* stream);
+
+/* y = y * silu(z), RMS-normed in `parts` equal parts of a row, times w: in place, y [T, parts * size], rows of z z_stride
+ * elements apart, w float32 [parts * size]. */
+int ed_gated_norm(void* y, const void* z, int64_t z_stride, const float* w, int64_t T, int parts, int size, double eps, int dtype,
+                  void* stream);
+
 /* out = act(x w^T) for a decode batch, bf16 operands: x [T, K], w [N, K], T <= 64 (fewer for large
  * weights), K a multiple of 64; act 0: none,
- * 1: max(v, 0)^2.  splits > 1: out is float32 [splits, T, N], partial sums over K (no act).  ed_skinny_gemm_splits: how
+ * 1: max(v, 0)^2, 2: w is [2 N, K], out = silu(x w_c) * (x w_(N + c)) in bf16.  splits > 1: out is float32 [splits, T, N], partial sums over K (no act).  ed_skinny_gemm_splits: how
  * many fill the chip, 0 if the shape is not taken. */
 int ed_skinny_gemm_splits(int64_t T, int N, int K);
 int ed_skinny_gemm(const void* x, const void* w, void* out, int out_dtype, int splits, int64_t T, int N, int K, int act,
@@ -90,6 +99,83 @@ typedef struct ed_gla_args {
 int ed_gla_prefill(const ed_gla_args* a, void* stream);
 /* One token per sequence: row s belongs to sequence s. */
 int ed_gla_step(const ed_gla_args* a, void* stream);
+
+/*
+ * Recurrences with one decay per head and token, behind short causal convolutions:
+ *   S <- g S;  u = beta (v - S^T k) (delta rule), or beta v (additive rule: beta_in is null);  S <- S + k u^T;  o = S^T q
+ * with a float32 state S [dim, vdim] per head; query/key head of head h: h / (heads / kv_heads).
+ * log g = -exp(a_log) softplus(decay_in + dt_bias).  Delta rule: beta = sigmoid(beta_in), and o is RMS-normed per head
+ * with norm_w and multiplied by silu(gate).  Additive rule: beta is that softplus, and skip * v is added to o (skip may be
+ * null).  q, k, v are silu(sum_j conv_w[., j] x_(t - taps + 1 + j) + conv_b) of the projections; with unit_eps > 0, q and k
+ * are then divided by sqrt(sum of squares + unit_eps); q is multiplied by q_scale.
+ * q, k: head g at g * dim of a row; v, gate: head h at h * vdim; decay_in, beta_in: column h; all rows `stride` elements
+ * apart.  dim, vdim <= 256, taps <= 16.
+ * ring: the last projections of every sequence, [slots, taps, channels] in the compute type, position p in row p % taps,
+ * channels = q, k, v one behind the other, as in conv_w and conv_b.  A sequence with starts[s] == 0 begins with zeros,
+ * whatever its slot holds.
+ */
+typedef struct ed_recur_args {
+    const void *q, *k, *v, *decay_in, *beta_in, *gate;
+    int64_t stride;
+    const float *conv_w, *conv_b, *a_log, *dt_bias, *skip, *norm_w;
+    void* ring;
+    float* states;             /* [slots, heads, dim, vdim] */
+    void* out;                 /* [T, heads * vdim] */
+    const int32_t *slots, *starts; /* [n_seqs] */
+    /* prompts only: */
+    const int32_t *q_begin;    /* [n_seqs + 1] */
+    const int32_t *chunks, *seq_chunks; /* as for ed_gla_prefill */
+    float *q_rows, *k_rows;    /* [T, kv_heads, round_up(dim, 16)] scratch */
+    void* v_rows;              /* [T, heads * vdim] scratch, compute type */
+    float* rates;              /* [T, heads, 2] scratch */
+    float* blocks;             /* [n_chunks, chunk_tokens / 16, heads, ed_recur_record(delta)] scratch */
+    float* chunk_states;       /* [n_chunks, heads, dim, vdim] scratch, null if every sequence has one chunk */
+    float* chunk_trans;        /* [n_chunks, heads, round_up(dim, 16)^2] (delta) or [n_chunks, heads] scratch, null likewise */
+    int32_t n_seqs, n_chunks, chunk_tokens /* a multiple of 16 */;
+    int32_t heads, kv_heads, dim, vdim, taps, dtype;
+    float q_scale, unit_eps, eps;
+} ed_recur_args;
+
+int ed_recur_record(int delta);
+/* Portions of prompts: any number of tokens per sequence. */
+int ed_recur_prefill(const ed_recur_args* a, void* stream);
+/* One token per sequence: row s belongs to sequence s. */
+int ed_recur_step(const ed_recur_args* a, void* stream);
+
+/*
+ * Softmax attention over a paged cache, query head h on key/value head h / (heads / kv_heads).  A token's cache row holds
+ * kv_heads keys of round_up(dim, 8) elements and behind them kv_heads values of round_up(vdim, 8) (ed_attn_row_elems in
+ * all), zeros in the padding; key j of sequence s is row tables[s][j / block_size] * block_size + j % block_size.
+ * dim, vdim <= 256, rot even and <= dim.
+ */
+typedef struct ed_attn_args {
+    const void *q, *k, *v;     /* projections, rows `stride` apart, heads next to each other */
+    int64_t stride;
+    const void* v_first;       /* rows v_first_stride apart: v becomes (1 - *mix) v + *mix v_first; null with mix */
+    int64_t v_first_stride;
+    const float* mix;
+    const float *q_norm, *k_norm; /* [dim] weights of the heads' RMS norms, or null */
+    const float* inv_freq;     /* [rot / 2]: pair (2i, 2i + 1) of the first rot elements turns by position * inv_freq[i] */
+    const int32_t *positions, *cache_rows; /* [T] */
+    void* cache;
+    void* q_rows;              /* [T, heads, round_up(dim, 8)] scratch: queries, normed and rotated */
+    void* out;                 /* [T, heads * vdim] */
+    const int32_t *q_begin, *starts, *tables; /* [n_seqs + 1], [n_seqs], [n_seqs, table_width] */
+    float *part_o, *part_ml;   /* [T * heads, splits, vdim], [T * heads, splits, 2] scratch, unused if splits == 1 */
+    int64_t T;
+    int32_t n_seqs, max_q, table_width, block_size, splits;
+    int32_t heads, kv_heads, dim, vdim, rot, window /* keys a query sees, itself included; 0: all */, dtype;
+    float scale, softcap /* score = softcap tanh(score / softcap); 0: none */, eps;
+} ed_attn_args;
+
+int ed_attn_row_elems(int kv_heads, int dim, int vdim);
+/* Norms, rotation and mixing: keys and values into the cache, queries into q_rows. */
+int ed_attn_prepare(const ed_attn_args* a, void* stream);
+/* Any portions; the keys of a row are shared out over `splits` (<= 64) workgroups. */
+int ed_attn_paged(const ed_attn_args* a, void* stream);
+/* Long portions, bf16: the same result (see ed_attn_prompt_supported). */
+int ed_attn_prompt_supported(int dim, int vdim);
+int ed_attn_prompt(const ed_attn_args* a, void* stream);
 
 /*
  * Latent attention.  The cache holds, per token, round_up(rank, 8) elements of the normed latent and round_up(rot, 8) of
