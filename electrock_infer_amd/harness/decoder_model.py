@@ -35,8 +35,10 @@ class DecoderModel(nn.Module):
             return None
         prefix, layer = f"layers.{first[1:]}.", self.layers[int(first[1:])]
         part, _, inner = rest.partition(".")
-        module = getattr(layer, part, None) if inner else None
-        if module is not None and hasattr(module, "TENSORS"):
+        module = getattr(layer, part, None) if inner else layer
+        if module is None:
+            return None
+        if inner and hasattr(module, "TENSORS"):
             entry = module.TENSORS.get(inner)
             return (f"{prefix}{part}.{entry[0]}", entry[1]) if entry is not None else None
         return prefix + rest, None
