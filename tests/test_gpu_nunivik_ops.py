@@ -128,7 +128,7 @@ def test_attention_prompts_steps_and_portions(entry, dtype):
         close(torch.cat([parts[0][i]] + ([parts[1][i - 1]] if i >= 1 else [])), ref, dtype, bf16=3e-2)
 
 
-def planted(entry, n, key, seed=1, strength=6.0):
+def planted(entry, n, key, seed=1, strength=1.0):
     """Hidden rows and weights for which the last query's score with one key stands out from all others: of a row, the first
     part makes queries, the second keys and the third values (no rotation)."""
     m = entry["mixer"]
@@ -336,7 +336,7 @@ def test_recurrence_over_many_chunks_in_a_batch():
         parts = [feed.step(mix, cache, [10, 0, 64, 1, 0], F32), feed.step(mix, cache, [200, 20, 64, 64, 1], F32)]
         first = {0: parts[0][0], 2: parts[0][1], 3: parts[0][2]}
         for i, ref in enumerate(want):
-            close(torch.cat([first[i]] * (i in first) + [parts[1][i]]), ref, F32, f32=1e-4)
+            close(torch.cat([first[i], parts[1][i]] if i in first else [parts[1][i]]), ref, F32, f32=1e-4)
 
 
 def test_convolution_windows_at_the_borders_of_portions():
