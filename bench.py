@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the Mixtral MoE layer on one MI355X.
 
-    python bench.py --model feguvik [--decoder-sizes 2048,4096]     (decoder models side by side; see decoder_rows)
+    python bench.py --model feguvik|nunivik [--decoder-sizes 2048,4096]     (decoder models side by side; see decoder_rows)
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--tokens T] [--shape 8x7b|8x22b] [--mode MODE]
                     [--routing normal|zipf|two_experts|balanced] [--no-cpu] [--no-table] [--no-e2e] [--detail FILE]
 
@@ -104,12 +104,13 @@ def parse_args():
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="first run three device copies of 1 GiB (a plain copy kernel of known size that the "
                          "FETCH_SIZE / WRITE_SIZE counters of a rocprofv3 --pmc run are scaled by)")
-    ap.add_argument("--model", choices=["mixtral-moe-layer", "feguvik"], default="mixtral-moe-layer",
+    ap.add_argument("--model", choices=["mixtral-moe-layer", "feguvik", "nunivik"], default="mixtral-moe-layer",
                     help="feguvik: prefill and decode throughput of Feguvik models through the engine's runner, next to "
-                         "Mixtral models of equal size, instead of the MoE layer benchmark")
-    ap.add_argument("--decoder-sizes", default="2048,4096", help="widths of the --model feguvik rows")
-    ap.add_argument("--decoder-only", choices=["feguvik", "mixtral"], default=None,
-                    help="run one of the two models of the --model feguvik rows (profiling)")
+                         "Mixtral models of equal size, instead of the MoE layer benchmark; nunivik: of Nunivik models, "
+                         "next to Feguvik models of equal size")
+    ap.add_argument("--decoder-sizes", default="2048,4096", help="widths of the decoder models")
+    ap.add_argument("--decoder-only", choices=["feguvik", "mixtral", "nunivik"], default=None,
+                    help="run one of the two decoder models (profiling)")
     ap.add_argument("--detail", default=None, help="write the unabridged measurements to this JSON file")
     return ap.parse_args()
 
@@ -428,20 +429,30 @@ def compact_e2e(r):
 
 
 # ---- decoder models through the engine's runner ----
-def decoder_configs(width):
-    """A Feguvik model and a Mixtral model of equal width, heads, layer runs and active feed-forward flops (two of eight
-    experts with three matrices of I rows = a dense feed-forward with two matrices of 3 I rows)."""
-    from electrock_infer_amd.harness import FeguvikConfig, ModelConfig
+def decoder_configs(width, model="feguvik"):
+    """Two models of equal width, heads and layer runs.  A Feguvik model and a Mixtral model of equal active feed-forward
+    flops (two of eight experts with three matrices of I rows = a dense feed-forward with two matrices of 3 I rows); or a
+    Nunivik model (a gated feed-forward: three matrices of 2 I rows) and that Feguvik model."""
+    from electrock_infer_amd.harness import FeguvikConfig, ModelConfig, NunivikConfig
     from electrock_infer_amd.harness.feguvik import LayerSpec, LoopSpec
+    from electrock_infer_amd.harness.nunivik import MixerSpec
     heads = width // 128
     gla = LayerSpec("gla", {"heads": heads, "dim": 64, "vdim": 128, "tau": 16.0}, 3 * width, decay_rank=16)
     mla = LayerSpec("latent_attention", {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512,
                                          "rot": {"base": 10000.0, "dims": 64}, "scale": 192 ** -0.5}, 3 * width)
     feg = FeguvikConfig(vocab_size=32000, width=width, layers=[gla, mla, gla, mla, gla, mla], norm_eps=1e-6,
                         embedding_scale=1.0, side_dim=64, loop=LoopSpec(1, 3, 2))
-    mix = ModelConfig(vocab_size=32000, hidden_size=width, intermediate_size=width, num_hidden_layers=8,
-                      num_attention_heads=heads, num_key_value_heads=max(heads // 4, 1))
-    return {"feguvik": feg, "mixtral": mix}
+    if model == "feguvik":
+        mix = ModelConfig(vocab_size=32000, hidden_size=width, intermediate_size=width, num_hidden_layers=8,
+                          num_attention_heads=heads, num_key_value_heads=max(heads // 4, 1))
+        return {"feguvik": feg, "mixtral": mix}
+    attention = {"heads": heads, "kv_heads": max(heads // 4, 1), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+                 "v_mix": True, "rot": {"base": 10000.0, "dims": 128, "scaling": {"factor": 2.0}}}
+    layers = [MixerSpec("delta", {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}, 2 * width),
+              MixerSpec("attention", attention, 2 * width),
+              MixerSpec("mamba2", {"heads": 2 * width // 64, "groups": 1, "state": 128, "vdim": 64, "conv": 4, "norm_groups": 1}, 2 * width),
+              MixerSpec("attention", {**attention, "mask": {"size": 1024}}, 2 * width)]
+    return {"nunivik": NunivikConfig(vocab_size=32000, width=width, layers=layers * 2, norm_eps=1e-6), "feguvik": feg}
 
 
 def decoder_rows(torch, name, cfg, width, steps, warmup):
@@ -499,7 +510,7 @@ def decoder_rows(torch, name, cfg, width, steps, warmup):
 def decoder_bench(torch, args):
     rows = []
     for width in [int(w) for w in args.decoder_sizes.split(",")]:
-        for name, cfg in decoder_configs(width).items():
+        for name, cfg in decoder_configs(width, args.model).items():
             if args.decoder_only in (None, name):
                 rows += decoder_rows(torch, name, cfg, width, min(args.steps, 10), min(args.warmup, 3))
                 print(f"[decoder] {name} width {width} done", file=sys.stderr, flush=True)
@@ -526,7 +537,7 @@ def main():
         print("bench.py needs a GPU", file=sys.stderr)
         sys.exit(1)
     from electrock_infer_amd import _lib
-    if args.model == "feguvik":
+    if args.model != "mixtral-moe-layer":
         return decoder_bench(torch, args)
     _lib.load()
     dev = torch.device("cuda:0")

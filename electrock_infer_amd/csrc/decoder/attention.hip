@@ -29,8 +29,8 @@ __device__ __forceinline__ float wave_sum(float v) {
 }
 
 // ---- norms, rotation, mixing, cache write ----
-// One workgroup per token, a wave per head.
-template <typename Elem>
+// One workgroup, or for few tokens several, per token; a wave per head.  PAIR: heads begin at a multiple of two elements.
+template <typename Elem, bool PAIR>
 __global__ __launch_bounds__(256) void attn_prepare_kernel(AttnProblem p) {
     typedef typename Elem::storage S;
     constexpr int kPairs = 2;        // per lane: heads of up to 256 elements
@@ -47,7 +47,7 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(AttnProblem p) {
     __syncthreads();
     const int dp = attn_pitch(dim), vp = attn_pitch(p.vdim), row = attn_row_elems(p.kv_heads, dim, p.vdim);
     S* cached = static_cast<S*>(p.cache) + static_cast<int64_t>(p.cache_rows[t]) * row;
-    for (int u = tid >> 6; u < p.heads + p.kv_heads; u += 4) {
+    for (int u = blockIdx.y * 4 + (tid >> 6); u < p.heads + p.kv_heads; u += 4 * gridDim.y) {
         const bool is_q = u < p.heads;
         const int h = is_q ? u : u - p.heads;
         const S* src = static_cast<const S*>(is_q ? p.q : p.k) + t * p.stride + h * dim;
@@ -57,8 +57,15 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(AttnProblem p) {
 #pragma unroll
         for (int i = 0; i < kPairs; ++i) {
             const int c = (lane + i * kWave) * 2;
-            a[i] = c < dim ? Elem::load(src[c]) : 0.0f;
-            b[i] = c + 1 < dim ? Elem::load(src[c + 1]) : 0.0f;
+            if (PAIR) {
+                S two[2] = {0, 0};
+                if (c < dim) __builtin_memcpy(two, __builtin_assume_aligned(src + c, sizeof(two)), sizeof(two));
+                a[i] = Elem::load(two[0]);
+                b[i] = Elem::load(two[1]);
+            } else {
+                a[i] = c < dim ? Elem::load(src[c]) : 0.0f;
+                b[i] = c + 1 < dim ? Elem::load(src[c + 1]) : 0.0f;
+            }
             ss = fmaf(a[i], a[i], fmaf(b[i], b[i], ss));
         }
         if (w != nullptr) {
@@ -85,7 +92,7 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(AttnProblem p) {
     }
     const float lambda = p.mix != nullptr ? *p.mix : 0.0f;
     S* values = cached + p.kv_heads * dp;
-    for (int i = tid; i < p.kv_heads * vp; i += 256) {
+    for (int i = blockIdx.y * 256 + tid; i < p.kv_heads * vp; i += 256 * gridDim.y) {
         const int g = i / vp, c = i - g * vp;
         float v = 0.0f;
         if (c < p.vdim) {
@@ -566,10 +573,17 @@ bool attn_supported(int heads, int kv_heads, int dim, int vdim, int rot) {
 }
 
 int launch_attn_prepare(const AttnProblem& p, int64_t T, hipStream_t s) {
-    const dim3 grid(static_cast<unsigned>(T));
+    const dim3 grid(static_cast<unsigned>(T), T <= 256 ? static_cast<unsigned>(ceil_div(p.heads + p.kv_heads, 4)) : 1u);
     const size_t lds = sizeof(float) * (p.rot > 0 ? p.rot : 1);
-    if (p.dtype == EM_DTYPE_BF16) launch((attn_prepare_kernel<BF16Elem>), grid, dim3(256), lds, s, p);
-    else launch((attn_prepare_kernel<F32Elem>), grid, dim3(256), lds, s, p);
+    const size_t two = 2 * (p.dtype == EM_DTYPE_BF16 ? 2 : 4);
+    const bool pair = p.dim % 2 == 0 && p.stride % 2 == 0 && reinterpret_cast<uintptr_t>(p.q) % two == 0 && reinterpret_cast<uintptr_t>(p.k) % two == 0;
+    if (p.dtype == EM_DTYPE_BF16) {
+        if (pair) launch((attn_prepare_kernel<BF16Elem, true>), grid, dim3(256), lds, s, p);
+        else launch((attn_prepare_kernel<BF16Elem, false>), grid, dim3(256), lds, s, p);
+    } else {
+        if (pair) launch((attn_prepare_kernel<F32Elem, true>), grid, dim3(256), lds, s, p);
+        else launch((attn_prepare_kernel<F32Elem, false>), grid, dim3(256), lds, s, p);
+    }
     return launch_status();
 }
 

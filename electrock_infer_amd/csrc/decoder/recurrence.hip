@@ -39,6 +39,8 @@ constexpr int kRecScores = 0, kRecDecay = 256, kRecRest = 272, kRecBeta = 288, k
 static_assert(recur_record(false) == kRecInverse && recur_record(true) == kRecInverse + 256, "a block's record");
 
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
+// with the hardware's exponential, reciprocal and square root, 1 ulp each
+__device__ __forceinline__ float silu_fast(float g) { return g * __builtin_amdgcn_rcpf(1.0f + exp2_fast(-g * kLog2e)); }
 __device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 
@@ -76,10 +78,11 @@ __device__ __forceinline__ void load_channels(const typename Elem::storage* src,
 }
 
 // ---- prompts: convolutions, unit vectors, decays ----
-// A wave takes 16 tokens of one q or k head or of kConvPiece channels of v; the last wave's share is decays and betas.
-// K >= taps: rows that a lane keeps.  VEC: all counts and offsets are multiples of four.
+// A wave takes 16 tokens of kConvPiece channels: four per lane, of as many q or k heads as fit (a head has a power of two of
+// lanes, `head_lanes`) or of v; the last wave's share is decays and betas.  K >= taps: rows that a lane keeps.  VEC: all
+// counts and offsets are multiples of four.
 template <typename Elem, int K, bool VEC>
-__global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p) {
+__global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p, int head_lanes) {
     typedef typename Elem::storage S;
     const int4 ch = p.chunks[blockIdx.x];
     const int first = blockIdx.y * kBlock;
@@ -91,30 +94,29 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p) {
     const int start = p.starts[seq], pos0 = start + at0;
     const int lane = threadIdx.x & 63;
     const int v_count = p.heads * p.vdim, v_units = (v_count + kConvPiece - 1) / kConvPiece;
+    const int fit = kWave / head_lanes, head_units = (p.kv_heads + fit - 1) / fit;
     const int unit = blockIdx.z * 4 + (threadIdx.x >> 6);
-    if (unit > 2 * p.kv_heads + v_units) return;
-    if (unit == 2 * p.kv_heads + v_units) {
+    if (unit > 2 * head_units + v_units) return;
+    if (unit == 2 * head_units + v_units) {
         for (int i = lane; i < n * p.heads; i += kWave) {
             const int t = i / p.heads, h = i - t * p.heads;
             *reinterpret_cast<f32x2_t*>(p.rates + ((row0 + t) * p.heads + h) * 2) = decay_and_beta<Elem>(p, row0 + t, h);
         }
         return;
     }
-    const bool is_v = unit >= 2 * p.kv_heads, is_q = unit < p.kv_heads;
-    const int piece = is_v ? unit - 2 * p.kv_heads : is_q ? unit : unit - p.kv_heads;
-    const int size = is_v ? kConvPiece : p.dim;
-    const int count = is_v ? min(kConvPiece, v_count - piece * kConvPiece) : p.dim;
-    const S* src = static_cast<const S*>(is_v ? p.v : is_q ? p.q : p.k) + piece * size;
-    const int c = lane * 4;
+    const bool is_v = unit >= 2 * head_units, is_q = unit < head_units;
+    const int g = is_v ? 0 : (is_q ? unit : unit - head_units) * fit + lane / head_lanes;      // this lane's q or k head
+    const int begin = is_v ? (unit - 2 * head_units) * kConvPiece : g * p.dim;
+    const int count = is_v ? min(kConvPiece, v_count - begin) : g < p.kv_heads ? p.dim : 0;
+    const S* src = static_cast<const S*>(is_v ? p.v : is_q ? p.q : p.k) + begin;
+    const int c = (is_v ? lane : lane % head_lanes) * 4;
     const int channels = 2 * p.kv_heads * p.dim + v_count;
-    const int channel0 = (is_v ? 2 * p.kv_heads * p.dim : is_q ? 0 : p.kv_heads * p.dim) + piece * size;
+    const int channel0 = (is_v ? 2 * p.kv_heads * p.dim : is_q ? 0 : p.kv_heads * p.dim) + begin;
     S* ring = static_cast<S*>(p.ring) + static_cast<int64_t>(p.slots[seq]) * p.taps * channels + channel0;
 
     float cur[kBlock][4];
 #pragma unroll
-    for (int t = 0; t < kBlock; ++t) {
-        if (t < n) load_channels<Elem, VEC>(src + (row0 + t) * p.stride, c, count, cur[t]);
-    }
+    for (int t = 0; t < kBlock; ++t) load_channels<Elem, VEC>(src + (row0 + min(t, n - 1)) * p.stride, c, count, cur[t]);
     float w[K][4], bias[4];                                     // w[i]: of the row K - 1 - i tokens back
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -137,7 +139,6 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p) {
     const int dp = (p.dim + 15) / 16 * 16;
 #pragma unroll
     for (int t = 0; t < kBlock; ++t) {
-        if (t >= n) break;
         float y[4], ss = 0.0f;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
@@ -147,14 +148,14 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p) {
                 y[j] = fmaf(w[i][j], hist[i][j], y[j]);
                 hist[i][j] = i + 1 < K - 1 ? hist[i + 1][j] : cur[t][j];
             }
-            y[j] = silu(fmaf(w[K - 1][j], cur[t][j], y[j]));
+            y[j] = silu_fast(fmaf(w[K - 1][j], cur[t][j], y[j]));
             ss = fmaf(y[j], y[j], ss);
         }
         const int64_t row = row0 + t;
         if (is_v) {
-            S* dst = static_cast<S*>(p.v_f) + row * v_count + piece * size;
+            S* dst = static_cast<S*>(p.v_f) + row * v_count + begin;
             if (VEC) {
-                if (c < count) {
+                if (c < count && t < n) {
                     S s4[4];
 #pragma unroll
                     for (int j = 0; j < 4; ++j) s4[j] = Elem::store(y[j]);
@@ -163,18 +164,21 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p) {
             } else {
 #pragma unroll
                 for (int j = 0; j < 4; ++j)
-                    if (c + j < count) dst[c + j] = Elem::store(y[j]);
+                    if (c + j < count && t < n) dst[c + j] = Elem::store(y[j]);
             }
         } else {
             float scale = is_q ? p.q_scale : 1.0f;
-            if (p.unit_eps > 0.0f) scale /= sqrtf(wave_sum(ss) + p.unit_eps);
+            if (p.unit_eps > 0.0f) {
+                for (int off = head_lanes / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off);
+                scale *= __builtin_amdgcn_rsqf(ss + p.unit_eps);
+            }
             // (channels beyond dim are zero: their weights are)
-            float* dst = (is_q ? p.q_f : p.k_f) + (row * p.kv_heads + piece) * dp;
-            if (c < dp) *reinterpret_cast<f32x4_t*>(dst + c) = f32x4_t{y[0] * scale, y[1] * scale, y[2] * scale, y[3] * scale};
+            float* dst = (is_q ? p.q_f : p.k_f) + (row * p.kv_heads + g) * dp;
+            if (c < dp && count > 0 && t < n) *reinterpret_cast<f32x4_t*>(dst + c) = f32x4_t{y[0] * scale, y[1] * scale, y[2] * scale, y[3] * scale};
         }
     }
     if (at0 != 0) return;
-    // (the wave that reads the ring's old rows of these channels is the one that replaces them)
+    // (the lane that reads the ring's old rows of these channels is the one that replaces them)
     for (int back = min(p.taps - 1, n_seq); back > 0; --back) {
         const int64_t row = static_cast<int64_t>(q_begin) + n_seq - back;
         S* dst = ring + static_cast<int64_t>((start + n_seq - back) % p.taps) * channels;
@@ -185,24 +189,26 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p) {
 }
 
 // ---- prompts: every block's scores and inverse ----
-// A wave takes one (block, head).
+// A wave takes one block and up to kBlockHeads of the heads that share q and k.
+constexpr int kBlockHeads = 8;
 template <bool DELTA>
-__global__ __launch_bounds__(256) void recur_block_kernel(RecurProblem p) {
+__global__ __launch_bounds__(256) void recur_block_kernel(RecurProblem p, int heads_per_wave) {
     constexpr int kPitch = 20;
     __shared__ __attribute__((aligned(16))) float lds[4][kBlock * kPitch];
     const int4 ch = p.chunks[blockIdx.x];
     const int first = blockIdx.y * kBlock;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, l16 = lane & 15, lq = lane >> 4;
-    const int h = blockIdx.z * 4 + wave;
-    if (first >= ch.z || h >= p.heads) return;                  // (waves share nothing)
+    const int share = p.heads / p.kv_heads, h0 = (blockIdx.z * 4 + wave) * heads_per_wave;   // (a divisor of `share`)
+    if (first >= ch.z || h0 >= p.heads) return;                 // (waves share nothing)
     const int n = min(kBlock, ch.z - first);
     const int64_t row0 = static_cast<int64_t>(ch.y) + first;
-    const int dp = (p.dim + 15) / 16 * 16, g = h / (p.heads / p.kv_heads);
+    const int dp = (p.dim + 15) / 16 * 16, g = h0 / share;
     const int64_t pitch = static_cast<int64_t>(p.kv_heads) * dp;
     const bool ok = l16 < n;
     const float* kr = p.k_f + (row0 + (ok ? l16 : 0)) * pitch + g * dp + lq * 4;
     const float* qr = p.q_f + (row0 + (ok ? l16 : 0)) * pitch + g * dp + lq * 4;
     f32x4_t qk = {0.0f, 0.0f, 0.0f, 0.0f}, kk = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll 4
     for (int d = 0; d < dp; d += 16) {
         const f32x4_t q4 = *reinterpret_cast<const f32x4_t*>(qr + d), k4 = *reinterpret_cast<const f32x4_t*>(kr + d);
 #pragma unroll
@@ -211,50 +217,53 @@ __global__ __launch_bounds__(256) void recur_block_kernel(RecurProblem p) {
             if (DELTA) kk = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[r], k4[r], kk, 0, 0, 0);
         }
     }
-    f32x2_t rate = {0.0f, 0.0f};
-    if (ok) rate = *reinterpret_cast<const f32x2_t*>(p.rates + ((row0 + l16) * p.heads + h) * 2);
-    float bl = rate[0];
-#pragma unroll
-    for (int off = 1; off < kBlock; off <<= 1) {
-        const float up = __shfl_up(bl, off, kBlock);
-        if (l16 >= off) bl += up;
-    }
-    const float tot = __shfl(bl, kBlock - 1, kBlock);
     const int64_t nb = p.chunk_tokens / kBlock;
-    float* rec = p.blocks + ((blockIdx.x * nb + blockIdx.y) * p.heads + h) * recur_record(DELTA);
-    if (lq == 0) {
-        rec[kRecDecay + l16] = exp2_fast(bl);
-        rec[kRecRest + l16] = exp2_fast(tot - bl);
-        rec[kRecBeta + l16] = rate[1];
-        rec[kRecLog + l16] = tot;
-    }
     float* am = lds[wave];
+    for (int h = h0; h < h0 + heads_per_wave; ++h) {
+        f32x2_t rate = {0.0f, 0.0f};
+        if (ok) rate = *reinterpret_cast<const f32x2_t*>(p.rates + ((row0 + l16) * p.heads + h) * 2);
+        float bl = rate[0];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-        const int t = lq * 4 + r;
-        const float ratio = exp2_fast(fminf(__shfl(bl, t, kBlock) - bl, 0.0f)), beta = __shfl(rate[1], t, kBlock);
-        rec[kRecScores + t * kBlock + l16] = l16 <= t && t < n ? qk[r] * ratio : 0.0f;
-        if (DELTA) am[t * kPitch + l16] = l16 < t && t < n ? beta * kk[r] * ratio : 0.0f;
-    }
-    if (!DELTA) return;
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    // column l16 of the inverse of the unit lower triangular matrix, row by row (each quarter of the wave on its own)
-    float inv[kBlock];
-#pragma unroll
-    for (int t = 0; t < kBlock; ++t) {
-        float v = t == l16 ? 1.0f : 0.0f;
-#pragma unroll
-        for (int s0 = 0; s0 < t; s0 += 4) {
-            const f32x4_t a = *reinterpret_cast<const f32x4_t*>(am + t * kPitch + s0);
-#pragma unroll
-            for (int j = 0; j < 4; ++j)
-                if (s0 + j < t) v = fmaf(-a[j], inv[s0 + j], v);
+        for (int off = 1; off < kBlock; off <<= 1) {
+            const float up = __shfl_up(bl, off, kBlock);
+            if (l16 >= off) bl += up;
         }
-        inv[t] = v;
-    }
+        const float tot = __shfl(bl, kBlock - 1, kBlock);
+        float* rec = p.blocks + ((blockIdx.x * nb + blockIdx.y) * p.heads + h) * recur_record(DELTA);
+        if (lq == 0) {
+            rec[kRecDecay + l16] = exp2_fast(bl);
+            rec[kRecRest + l16] = exp2_fast(tot - bl);
+            rec[kRecBeta + l16] = rate[1];
+            rec[kRecLog + l16] = tot;
+        }
 #pragma unroll
-    for (int t = 0; t < kBlock; ++t)
-        if ((t >> 2) == lq) rec[kRecInverse + t * kBlock + l16] = inv[t] * rate[1];
+        for (int r = 0; r < 4; ++r) {
+            const int t = lq * 4 + r;
+            const float ratio = exp2_fast(fminf(__shfl(bl, t, kBlock) - bl, 0.0f)), beta = __shfl(rate[1], t, kBlock);
+            rec[kRecScores + t * kBlock + l16] = l16 <= t && t < n ? qk[r] * ratio : 0.0f;
+            if (DELTA) am[t * kPitch + l16] = l16 < t && t < n ? beta * kk[r] * ratio : 0.0f;
+        }
+        if (!DELTA) continue;
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        // column l16 of the inverse of the unit lower triangular matrix, row by row (each quarter of the wave on its own)
+        float inv[kBlock];
+#pragma unroll
+        for (int t = 0; t < kBlock; ++t) {
+            float v = t == l16 ? 1.0f : 0.0f;
+#pragma unroll
+            for (int s0 = 0; s0 < t; s0 += 4) {
+                const f32x4_t a = *reinterpret_cast<const f32x4_t*>(am + t * kPitch + s0);
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    if (s0 + j < t) v = fmaf(-a[j], inv[s0 + j], v);
+            }
+            inv[t] = v;
+        }
+#pragma unroll
+        for (int t = 0; t < kBlock; ++t)
+            if ((t >> 2) == lq) rec[kRecInverse + t * kBlock + l16] = inv[t] * rate[1];
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    }
 }
 
 // ---- prompts: a chunk's blocks, one after the other ----
@@ -309,7 +318,8 @@ __global__ __launch_bounds__(THREADS) void recur_chunk_kernel(RecurProblem p) {
 
     // a block's operands, in flight while the one before is computed
     f32x4_t rk[kPieces], rq[kPieces], scores, inverse, decay, rest, beta;
-    float block_decay, block_log, v[4], gt[4];
+    float block_decay, block_log;
+    S v[4], gt[4];                                    // (as stored: a conversion here would wait for the load)
     auto fetch = [&](int b) {
         const int n = min(kBlock, ch.z - b * kBlock);
         const int64_t row0 = static_cast<int64_t>(ch.y) + b * kBlock;
@@ -334,8 +344,8 @@ __global__ __launch_bounds__(THREADS) void recur_chunk_kernel(RecurProblem p) {
         for (int r = 0; r < 4; ++r) {
             const int t = lq * 4 + r;
             const bool ok = v_ok && t < n;
-            v[r] = ok ? Elem::load(vg[(row0 + t) * v_pitch]) : 0.0f;
-            if (OUTPUT && DELTA) gt[r] = ok ? Elem::load(gate[(row0 + t) * p.stride]) : 0.0f;
+            v[r] = ok ? vg[(row0 + t) * v_pitch] : S(0);
+            if (OUTPUT && DELTA) gt[r] = ok ? gate[(row0 + t) * p.stride] : S(0);
         }
     };
     // a block's results wait for the row sums of the other waves until the next barrier
@@ -350,8 +360,8 @@ __global__ __launch_bounds__(THREADS) void recur_chunk_kernel(RecurProblem p) {
         for (int r = 0; r < 4; ++r) {
             const int t = lq * 4 + r;
             if (v_ok && t < n) {
-                const float y = held[r] / sqrtf(ss[r] * inv_vdim + p.eps) * norm_w;
-                static_cast<S*>(p.out)[(row0 + t) * v_pitch + h * vdim + col] = Elem::store(y * silu(held_gate[r]));
+                const float y = held[r] * __builtin_amdgcn_rsqf(ss[r] * inv_vdim + p.eps) * norm_w;
+                static_cast<S*>(p.out)[(row0 + t) * v_pitch + h * vdim + col] = Elem::store(y * silu_fast(held_gate[r]));
             }
         }
     };
@@ -373,8 +383,8 @@ __global__ __launch_bounds__(THREADS) void recur_chunk_kernel(RecurProblem p) {
         float v_b[4], gt_b[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            v_b[r] = v[r];
-            gt_b[r] = gt[r];
+            v_b[r] = Elem::load(v[r]);
+            gt_b[r] = OUTPUT && DELTA ? Elem::load(gt[r]) : 0.0f;
         }
         log_sum += block_log;
         __syncthreads();              // (the block before last, in the same half, has been used)
@@ -502,13 +512,13 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(RecurProblem p) {
     *slot = state;
 }
 
-// Delta rule: by a matrix.  One workgroup per (16 state columns, head, sequence), one wave per 16 rows.
+// Delta rule: by a matrix.  One workgroup per (head, 16 state columns, sequence), one wave per 16 rows.
 template <int NDT>
 __global__ __launch_bounds__(NDT * kWave) void recur_matrix_scan_kernel(RecurProblem p) {
     constexpr int kPitch = 20;
     __shared__ float state[2][NDT * 16 * kPitch];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, lq = lane >> 4;
-    const int col = blockIdx.x * 16 + l16, h = blockIdx.y, s = blockIdx.z;
+    const int col = blockIdx.y * 16 + l16, h = blockIdx.x, s = blockIdx.z;   // (a head's workgroups share an L2)
     const int dim = p.dim, vdim = p.vdim, dp = (dim + 15) / 16 * 16;
     const int c0 = p.seq_chunks[s], c1 = p.seq_chunks[s + 1];
     const int64_t n = static_cast<int64_t>(dim) * vdim, pitch = static_cast<int64_t>(p.heads) * n;
@@ -519,7 +529,7 @@ __global__ __launch_bounds__(NDT * kWave) void recur_matrix_scan_kernel(RecurPro
     const bool has_rows = wave * 16 < dp, zero = p.starts[s] == 0;
     const float* mr = p.chunk_trans + h * m_size + static_cast<int64_t>(has_rows ? wave * 16 + l16 : 0) * dp + lq * 4;
     bool ok[4];
-    f32x4_t cur, add = {0.0f, 0.0f, 0.0f, 0.0f}, m4[NDT];
+    f32x4_t cur, add = {0.0f, 0.0f, 0.0f, 0.0f}, m4[NDT];     // (the next chunk's, in flight)
     auto fetch = [&](int c) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) add[r] = ok[r] ? cs[c * pitch + static_cast<int64_t>(row + r) * vdim + col] : 0.0f;
@@ -540,18 +550,20 @@ __global__ __launch_bounds__(NDT * kWave) void recur_matrix_scan_kernel(RecurPro
             buf[(row + r) * kPitch + l16] = cur[r];
             if (ok[r]) cs[c * pitch + static_cast<int64_t>(row + r) * vdim + col] = cur[r];
         }
+        f32x4_t sum[2] = {add, f32x4_t{0.0f, 0.0f, 0.0f, 0.0f}}, now[NDT];
+#pragma unroll
+        for (int k = 0; k < NDT; ++k) now[k] = m4[k];
+        if (c + 1 < c1) fetch(c + 1);
         __syncthreads();
-        f32x4_t next = add;
 #pragma unroll
         for (int k = 0; k < NDT; ++k) {
             if (k < k_tiles) {
 #pragma unroll
                 for (int r = 0; r < 4; ++r)
-                    next = __builtin_amdgcn_mfma_f32_16x16x4f32(m4[k][r], buf[(k * 16 + lq * 4 + r) * kPitch + l16], next, 0, 0, 0);
+                    sum[r & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(now[k][r], buf[(k * 16 + lq * 4 + r) * kPitch + l16], sum[r & 1], 0, 0, 0);
             }
         }
-        cur = next;
-        if (c + 1 < c1) fetch(c + 1);
+        cur = sum[0] + sum[1];
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r)
@@ -693,14 +705,15 @@ __global__ __launch_bounds__(1024) void recur_step_kernel(RecurProblem p) {
 // ---- launches ----
 template <typename Elem>
 int launch_conv(const RecurProblem& p, hipStream_t s) {
-    const int v_units = static_cast<int>(ceil_div(p.heads * p.vdim, kConvPiece));
-    const dim3 grid(static_cast<unsigned>(p.n_chunks), static_cast<unsigned>(p.chunk_tokens / kBlock),
-                    static_cast<unsigned>(ceil_div(2 * p.kv_heads + v_units + 1, 4)));
+    int head_lanes = 1;
+    while (head_lanes * 4 < round_up(p.dim, 16)) head_lanes *= 2;
+    const int units = static_cast<int>(2 * ceil_div(p.kv_heads, kWave / head_lanes) + ceil_div(p.heads * p.vdim, kConvPiece) + 1);
+    const dim3 grid(static_cast<unsigned>(p.n_chunks), static_cast<unsigned>(p.chunk_tokens / kBlock), static_cast<unsigned>(ceil_div(units, 4)));
     auto aligned = [](const void* ptr) { return reinterpret_cast<uintptr_t>(ptr) % (4 * sizeof(typename Elem::storage)) == 0; };
     const bool vec = p.dim % 4 == 0 && p.vdim % 4 == 0 && p.stride % 4 == 0 && aligned(p.q) && aligned(p.k) && aligned(p.v);
-    if (p.taps > 4) launch((recur_conv_kernel<Elem, kMaxTaps, false>), grid, dim3(256), 0, s, p);
-    else if (vec) launch((recur_conv_kernel<Elem, 4, true>), grid, dim3(256), 0, s, p);
-    else launch((recur_conv_kernel<Elem, 4, false>), grid, dim3(256), 0, s, p);
+    if (p.taps > 4) launch((recur_conv_kernel<Elem, kMaxTaps, false>), grid, dim3(256), 0, s, p, head_lanes);
+    else if (vec) launch((recur_conv_kernel<Elem, 4, true>), grid, dim3(256), 0, s, p, head_lanes);
+    else launch((recur_conv_kernel<Elem, 4, false>), grid, dim3(256), 0, s, p, head_lanes);
     return launch_status();
 }
 
@@ -740,7 +753,7 @@ int launch_scan(const RecurProblem& p, hipStream_t s) {
         launch(recur_scan_kernel, dim3(static_cast<unsigned>(ceil_div(p.dim * p.vdim, 256)), heads, seqs), dim3(256), 0, s, p);
         return launch_status();
     }
-    const dim3 grid(static_cast<unsigned>(ceil_div(p.vdim, 16)), heads, seqs);
+    const dim3 grid(heads, static_cast<unsigned>(ceil_div(p.vdim, 16)), seqs);
     if (p.dim <= 32) launch(recur_matrix_scan_kernel<2>, grid, dim3(2 * kWave), 0, s, p);
     else if (p.dim <= 64) launch(recur_matrix_scan_kernel<4>, grid, dim3(4 * kWave), 0, s, p);
     else if (p.dim <= 128) launch(recur_matrix_scan_kernel<8>, grid, dim3(8 * kWave), 0, s, p);
@@ -752,8 +765,10 @@ template <typename Elem, bool DELTA>
 int prefill(const RecurProblem& p, hipStream_t s) {
     int rc = launch_conv<Elem>(p, s);
     if (rc != 0) return rc;
+    int per_wave = kBlockHeads;
+    while (p.heads / p.kv_heads % per_wave != 0) --per_wave;
     launch(recur_block_kernel<DELTA>, dim3(static_cast<unsigned>(p.n_chunks), static_cast<unsigned>(p.chunk_tokens / kBlock),
-                                           static_cast<unsigned>(ceil_div(p.heads, 4))), dim3(256), 0, s, p);
+                                           static_cast<unsigned>(ceil_div(p.heads / per_wave, 4))), dim3(256), 0, s, p, per_wave);
     rc = launch_status();
     if (rc != 0) return rc;
     if (p.chunk_states != nullptr) {

@@ -79,7 +79,7 @@ class DecodeGraphs:
 
     def _fill(self, seqs, padding: DecodePadding, into: Optional[RaggedBatch] = None) -> RaggedBatch:
         runner = self.runner
-        return make_ragged(seqs, runner.block_size, runner.model.CHUNK_TOKENS, runner.device, padding=padding, into=into)
+        return make_ragged(seqs, runner.block_size, runner.model.chunk_tokens(1), runner.device, padding=padding, into=into)
 
     # (outside inference mode: a recording leaves tensors behind in torch's generator that later recordings write to)
     @torch.inference_mode(False)

@@ -13,7 +13,6 @@ from .batch import RaggedBatch
 class DecoderModel(nn.Module):
 
     ragged_batches = True
-    CHUNK_TOKENS = 256        # tokens that one workgroup of the recurrent mixers' prompt kernels takes
     NAMES = {"embed": "embed", "final.norm": "final_norm", "head": "head"}     # tensors outside the layers
     ZEROS: Tuple[str, ...] = ()       # ends of vectors' names that random weights leave at zero (the others are ones)
 
@@ -24,6 +23,10 @@ class DecoderModel(nn.Module):
         super().__init__()
         self.caches: List = []            # per run: what its mixer's new_cache made
         self.layer_hook = None            # called as hook(run index, stream) behind every layer run when set
+
+    def chunk_tokens(self, tokens: int) -> int:
+        """Tokens that one workgroup of the recurrent mixers' prompt kernels takes in a step of ``tokens``."""
+        return 256
 
     # ---- weights ----
     def checkpoint_target(self, name: str):

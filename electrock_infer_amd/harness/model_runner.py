@@ -67,7 +67,8 @@ class ModelRunner:
         """The planned portions of any batch, for models that take RaggedBatch; ``rows``: batch rows whose logits are
         wanted (default: the last one of every sequence)."""
         self.check_slots(seqs)
-        return make_ragged(seqs, self.block_size, self.model.CHUNK_TOKENS, self.device, rows)
+        chunk = self.model.chunk_tokens(sum(s.num_scheduled_tokens for s in seqs))
+        return make_ragged(seqs, self.block_size, chunk, self.device, rows)
 
     def prepare_prefill(self, seqs: List[Sequence]):
         """Feed every sequence's planned portion behind its computed tokens; the cache slots follow from the block

@@ -114,6 +114,10 @@ class NunivikForCausalLM(DecoderModel):
         self.head = matrix(cfg.vocab_size, cfg.width)
         self.runs = [(i,) for i in range(len(cfg.layers))]
 
+    def chunk_tokens(self, tokens: int) -> int:
+        """Fewer, longer chunks where there are enough of them to fill the chip: the scan over them is sequential."""
+        return 512 if tokens >= 8192 else 256 if tokens >= 4096 else 128 if tokens >= 1024 else 64
+
     def forward(self, batch: RaggedBatch) -> torch.Tensor:
         """Normed output [T, width] of every token of the batch."""
         cfg, eps = self.cfg, self.cfg.norm_eps
