@@ -88,7 +88,7 @@ int check_recur(const ed_recur_args* a) {
     if (!a->q || !a->k || !a->v || !a->decay_in || (a->beta_in && (!a->gate || !a->norm_w)) || !a->conv_w || !a->a_log || !a->dt_bias ||
         !a->ring || !a->states || !a->out || !a->slots || !a->starts)
         return EM_ERR_NULL_POINTER;
-    if (!aligned16(a->states) || !aligned16(a->ring)) return EM_ERR_ALIGNMENT;
+    if (!aligned16(a->states) || !aligned16(a->ring) || !aligned16(a->conv_w)) return EM_ERR_ALIGNMENT;
     return 0;
 }
 

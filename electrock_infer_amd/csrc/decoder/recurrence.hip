@@ -79,7 +79,7 @@ __device__ __forceinline__ void load_channels(const typename Elem::storage* src,
 
 // ---- prompts: convolutions, unit vectors, decays ----
 // A wave takes 16 tokens of kConvPiece channels: four per lane, of as many q or k heads as fit (a head has a power of two of
-// lanes, `head_lanes`) or of v; the last wave's share is decays and betas.  K >= taps: rows that a lane keeps.  VEC: all
+// lanes, `head_lanes`) or of v; the last waves' share is decays and betas, one per lane.  K >= taps: rows that a lane keeps.  VEC: all
 // counts and offsets are multiples of four.
 template <typename Elem, int K, bool VEC>
 __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p, int head_lanes) {
@@ -96,12 +96,9 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p, int hea
     const int v_count = p.heads * p.vdim, v_units = (v_count + kConvPiece - 1) / kConvPiece;
     const int fit = kWave / head_lanes, head_units = (p.kv_heads + fit - 1) / fit;
     const int unit = blockIdx.z * 4 + (threadIdx.x >> 6);
-    if (unit > 2 * head_units + v_units) return;
-    if (unit == 2 * head_units + v_units) {
-        for (int i = lane; i < n * p.heads; i += kWave) {
-            const int t = i / p.heads, h = i - t * p.heads;
-            *reinterpret_cast<f32x2_t*>(p.rates + ((row0 + t) * p.heads + h) * 2) = decay_and_beta<Elem>(p, row0 + t, h);
-        }
+    if (unit >= 2 * head_units + v_units) {
+        const int i = (unit - 2 * head_units - v_units) * kWave + lane, t = i / p.heads, h = i - t * p.heads;
+        if (t < n) *reinterpret_cast<f32x2_t*>(p.rates + ((row0 + t) * p.heads + h) * 2) = decay_and_beta<Elem>(p, row0 + t, h);
         return;
     }
     const bool is_v = unit >= 2 * head_units, is_q = unit < head_units;
@@ -121,6 +118,13 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p, int hea
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
         bias[j] = p.conv_b != nullptr && c + j < count ? p.conv_b[channel0 + c + j] : 0.0f;
+        if (K == 4 && p.taps == 4) {
+            f32x4_t row = {0.0f, 0.0f, 0.0f, 0.0f};
+            if (c + j < count) row = *reinterpret_cast<const f32x4_t*>(p.conv_w + static_cast<int64_t>(channel0 + c + j) * 4);
+#pragma unroll
+            for (int i = 0; i < K; ++i) w[i][j] = row[i & 3];
+            continue;
+        }
 #pragma unroll
         for (int i = 0; i < K; ++i)
             w[i][j] = K - 1 - i < p.taps && c + j < count ? p.conv_w[static_cast<int64_t>(channel0 + c + j) * p.taps + p.taps - K + i] : 0.0f;
@@ -179,12 +183,19 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(RecurProblem p, int hea
     }
     if (at0 != 0) return;
     // (the lane that reads the ring's old rows of these channels is the one that replaces them)
-    for (int back = min(p.taps - 1, n_seq); back > 0; --back) {
-        const int64_t row = static_cast<int64_t>(q_begin) + n_seq - back;
+    S last[K][4];
+#pragma unroll
+    for (int back = 1; back < K; ++back)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+            last[back][j] = back < p.taps && back <= n_seq && c + j < count ? src[(static_cast<int64_t>(q_begin) + n_seq - back) * p.stride + c + j] : S(0);
+#pragma unroll
+    for (int back = 1; back < K; ++back) {
+        if (back >= p.taps || back > n_seq) continue;
         S* dst = ring + static_cast<int64_t>((start + n_seq - back) % p.taps) * channels;
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-            if (c + j < count) dst[c + j] = src[row * p.stride + c + j];
+            if (c + j < count) dst[c + j] = last[back][j];
     }
 }
 
@@ -515,8 +526,8 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(RecurProblem p) {
 // Delta rule: by a matrix.  One workgroup per (head, 16 state columns, sequence), one wave per 16 rows.
 template <int NDT>
 __global__ __launch_bounds__(NDT * kWave) void recur_matrix_scan_kernel(RecurProblem p) {
-    constexpr int kPitch = 20;
-    __shared__ float state[2][NDT * 16 * kPitch];
+    constexpr int kPitch = NDT * 16 + 4;
+    __shared__ __attribute__((aligned(16))) float state[2][16 * kPitch];      // column by column
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, lq = lane >> 4;
     const int col = blockIdx.y * 16 + l16, h = blockIdx.x, s = blockIdx.z;   // (a head's workgroups share an L2)
     const int dim = p.dim, vdim = p.vdim, dp = (dim + 15) / 16 * 16;
@@ -528,46 +539,61 @@ __global__ __launch_bounds__(NDT * kWave) void recur_matrix_scan_kernel(RecurPro
     const int row = wave * 16 + lq * 4, k_tiles = dp / 16;
     const bool has_rows = wave * 16 < dp, zero = p.starts[s] == 0;
     const float* mr = p.chunk_trans + h * m_size + static_cast<int64_t>(has_rows ? wave * 16 + l16 : 0) * dp + lq * 4;
+    // a chunk's matrix and contribution, in flight two chunks ahead (one, where the registers do not hold three matrices)
+    constexpr int kAhead = NDT <= 8 ? 2 : 1;
     bool ok[4];
-    f32x4_t cur, add = {0.0f, 0.0f, 0.0f, 0.0f}, m4[NDT];     // (the next chunk's, in flight)
-    auto fetch = [&](int c) {
+    f32x4_t cur, add[kAhead], m4[kAhead][NDT];
+    // (addresses are held inside instead of loads being skipped: waits can count straight-line loads)
+    int64_t from[4];
+    auto fetch = [&](int c, f32x4_t& to_add, f32x4_t (&to)[NDT]) {
+        c = min(c, c1 - 1);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) add[r] = ok[r] ? cs[c * pitch + static_cast<int64_t>(row + r) * vdim + col] : 0.0f;
+        for (int r = 0; r < 4; ++r) to_add[r] = cs[c * pitch + from[r]];
 #pragma unroll
-        for (int k = 0; k < NDT; ++k)
-            m4[k] = k < k_tiles ? *reinterpret_cast<const f32x4_t*>(mr + c * m_pitch + k * 16) : f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+        for (int k = 0; k < NDT; ++k) to[k] = *reinterpret_cast<const f32x4_t*>(mr + c * m_pitch + min(k, k_tiles - 1) * 16);
+    };
+    auto advance = [&](int c, f32x4_t& my_add, f32x4_t (&mine)[NDT]) {
+        float* buf = state[(c - c0) & 1];
+        *reinterpret_cast<f32x4_t*>(buf + l16 * kPitch + row) = cur;
+        f32x4_t sum[2] = {my_add, f32x4_t{0.0f, 0.0f, 0.0f, 0.0f}}, now[NDT];
+        if (kAhead == 2) {
+#pragma unroll
+            for (int k = 0; k < NDT; ++k) now[k] = mine[k];
+            fetch(c + 2, my_add, mine);
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+            if (ok[r]) cs[c * pitch + from[r]] = cur[r];
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < NDT; ++k) {
+            // (rows beyond dim are zero here, whatever stands in the matrix)
+            const f32x4_t s4 = *reinterpret_cast<const f32x4_t*>(buf + l16 * kPitch + k * 16 + lq * 4);
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                sum[r & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(kAhead == 2 ? now[k][r] : mine[k][r], s4[r], sum[r & 1], 0, 0, 0);
+        }
+        if (kAhead == 1) fetch(c + 1, my_add, mine);
+        cur = sum[0] + sum[1];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) cur[r] = ok[r] ? cur[r] : 0.0f;
     };
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         ok[r] = row + r < dim && col < vdim;
-        cur[r] = ok[r] && !zero ? slot[static_cast<int64_t>(row + r) * vdim + col] : 0.0f;
+        from[r] = ok[r] ? static_cast<int64_t>(row + r) * vdim + col : 0;
+        cur[r] = ok[r] && !zero ? slot[from[r]] : 0.0f;
     }
-    fetch(c0);
-    for (int c = c0; c < c1; ++c) {
-        float* buf = state[(c - c0) & 1];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            buf[(row + r) * kPitch + l16] = cur[r];
-            if (ok[r]) cs[c * pitch + static_cast<int64_t>(row + r) * vdim + col] = cur[r];
-        }
-        f32x4_t sum[2] = {add, f32x4_t{0.0f, 0.0f, 0.0f, 0.0f}}, now[NDT];
+    for (int i = 0; i < kAhead; ++i) fetch(c0 + i, add[i], m4[i]);
+    for (int c = c0; c < c1; c += kAhead) {
 #pragma unroll
-        for (int k = 0; k < NDT; ++k) now[k] = m4[k];
-        if (c + 1 < c1) fetch(c + 1);
-        __syncthreads();
-#pragma unroll
-        for (int k = 0; k < NDT; ++k) {
-            if (k < k_tiles) {
-#pragma unroll
-                for (int r = 0; r < 4; ++r)
-                    sum[r & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(now[k][r], buf[(k * 16 + lq * 4 + r) * kPitch + l16], sum[r & 1], 0, 0, 0);
-            }
-        }
-        cur = sum[0] + sum[1];
+        for (int i = 0; i < kAhead; ++i)
+            if (c + i < c1) advance(c + i, add[i], m4[i]);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-        if (ok[r]) slot[static_cast<int64_t>(row + r) * vdim + col] = cur[r];
+        if (ok[r]) slot[from[r]] = cur[r];
 }
 
 // ---- decoding: one new token per sequence ----
@@ -707,7 +733,7 @@ template <typename Elem>
 int launch_conv(const RecurProblem& p, hipStream_t s) {
     int head_lanes = 1;
     while (head_lanes * 4 < round_up(p.dim, 16)) head_lanes *= 2;
-    const int units = static_cast<int>(2 * ceil_div(p.kv_heads, kWave / head_lanes) + ceil_div(p.heads * p.vdim, kConvPiece) + 1);
+    const int units = static_cast<int>(2 * ceil_div(p.kv_heads, kWave / head_lanes) + ceil_div(p.heads * p.vdim, kConvPiece) + ceil_div(kBlock * p.heads, kWave));
     const dim3 grid(static_cast<unsigned>(p.n_chunks), static_cast<unsigned>(p.chunk_tokens / kBlock), static_cast<unsigned>(ceil_div(units, 4)));
     auto aligned = [](const void* ptr) { return reinterpret_cast<uintptr_t>(ptr) % (4 * sizeof(typename Elem::storage)) == 0; };
     const bool vec = p.dim % 4 == 0 && p.vdim % 4 == 0 && p.stride % 4 == 0 && aligned(p.q) && aligned(p.k) && aligned(p.v);
