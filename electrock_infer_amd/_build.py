@@ -1,8 +1,8 @@
 """Build recipe for libelectrock_moe.so and libelectrock_decoder.so (gfx950 only).
 
 Two libraries, so that a model compiles what it needs: csrc/*.hip is the MoE layer, csrc/decoder/*.hip the kernels of
-decoders with a float32 stream, gated linear attention and latent attention (no hand-counted copies there: the checks
-below are about the first one).
+decoders with a float32 stream, linear attention, recurrences, latent and softmax attention (no hand-counted copies
+there: the checks below are about the first one).
 
 The MoE library is compiled in-tree with plain hipcc; there is no CPU build of the
 kernels and no fallback: importing the ops without the built library fails.
